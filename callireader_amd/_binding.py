@@ -14,7 +14,7 @@ _LIB_PATH = os.environ.get('CR_HIP_LIB') or os.path.join(os.path.dirname(os.path
 
 CR_OK = 0
 CR_BF16, CR_F32, CR_I64, CR_I32 = 0, 1, 2, 3
-ABI_VERSION = 11
+ABI_VERSION = 12
 
 
 class ModelDesc(C.Structure):
@@ -23,18 +23,31 @@ class ModelDesc(C.Structure):
                 ('rms_eps', C.c_float), ('reserved', C.c_int32 * 8)]
 
 
+class LmHeads(C.Structure):
+    _fields_ = [('name', C.c_char * 16)] + [(n, C.c_int32) for n in ('heads', 'kv_heads', 'dim', 'vdim', 'chunk', 'qk_norm', 'rot_dims', 'reserved')] + \
+               [('rot_base', C.c_double)] + [(n, C.c_float) for n in ('scale', 'softcap', 'out_scale', 'reserved_f')]
+
+
+class LmRetention(C.Structure):
+    _fields_ = [('name', C.c_char * 16)] + [(n, C.c_int32) for n in ('heads', 'dim', 'vdim', 'rot_dims')] + \
+               [('rot_base', C.c_double), ('k_scale', C.c_float), ('out_scale', C.c_float), ('decay', C.POINTER(C.c_double))]
+
+
 class LmLayer(C.Structure):
     _fields_ = [(n, C.c_int32) for n in ('mixer', 'heads', 'dim', 'vdim', 'q_rank', 'kv_rank')] + [('scale', C.c_float)] + \
-               [(n, C.c_int32) for n in ('ff', 'experts', 'top', 'expert_ff', 'groups', 'keep')] + [('limit', C.c_float), ('reserved', C.c_int32 * 8)]
+               [(n, C.c_int32) for n in ('ff', 'experts', 'top', 'expert_ff', 'groups', 'keep')] + [('limit', C.c_float), ('act', C.c_int32), ('reserved', C.c_int32 * 7),
+                                                                                                    ('attn', LmHeads), ('ret', LmRetention)]
 
 
 class LmDesc(C.Structure):
     _fields_ = [(n, C.c_int32) for n in ('layers', 'width', 'vocab', 'dtype', 'loop_start', 'loop_stop', 'loop_times', 'pos')] + \
-               [(n, C.c_float) for n in ('pos_base', 'eps', 'softcap')] + [('reserved', C.c_int32 * 8)]
+               [(n, C.c_float) for n in ('pos_base', 'eps', 'softcap')] + \
+               [(n, C.c_int32) for n in ('norm_plain', 'no_post_norm', 'tied_head', 'loop_in', 'side_dim')] + [('reserved', C.c_int32 * 7)]
 
 
-CR_MIX_LATENT = 1
-CR_FF_NONE, CR_FF_MOE = 0, 1
+CR_MIX_LATENT, CR_MIX_HEADS, CR_MIX_RETENTION = 1, 2, 4
+CR_FF_NONE, CR_FF_MOE, CR_FF_DENSE = 0, 1, 2
+CR_ACT_RELU2 = 1
 CR_POS_NONE, CR_POS_SINUSOID = 0, 1
 
 vp, i32, i64, f32 = C.c_void_p, C.c_int, C.c_int64, C.c_float

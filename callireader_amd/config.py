@@ -137,6 +137,63 @@ class LatentMixer:
     kv_rank: int
     scale: float
 
+    def weight_shapes(self, p, W):
+        return {p + 'dq': (self.q_rank, W), p + 'dq.norm': (self.q_rank,), p + 'uq': (self.heads * self.dim, self.q_rank), p + 'dkv': (self.kv_rank, W), p + 'dkv.norm': (self.kv_rank,),
+                p + 'uk': (self.heads * self.dim, self.kv_rank), p + 'uv': (self.heads * self.vdim, self.kv_rank), p + 'g': (self.heads * self.vdim, W),
+                p + 'o': (W, self.heads * self.vdim)}
+
+
+@dataclass(frozen=True)
+class Rotation:
+    """Entries i and i + dims / 2 of a head turn by position * base^(-2 i / dims); entries from `dims` on stay."""
+    base: float
+    dims: int
+
+
+@dataclass(frozen=True)
+class HeadsMixer:
+    """Softmax attention over grouped heads (CR_MIX_HEADS); chunk: keys of the query's own chunk of positions only (0: every earlier key)."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    rot: Rotation = None
+    chunk: int = 0
+    softcap: float = 0.0
+    qk_norm: bool = False
+
+    def weight_shapes(self, p, W):
+        out = {p + 'q': (self.heads * self.dim, W), p + 'k': (self.kv_heads * self.dim, W), p + 'v': (self.kv_heads * self.vdim, W), p + 'o': (W, self.heads * self.vdim)}
+        return {**out, p + 'q.norm': (self.dim,), p + 'k.norm': (self.dim,)} if self.qk_norm else out
+
+
+@dataclass(frozen=True)
+class RetentionMixer:
+    """Linear attention with a fixed decay per head (CR_MIX_RETENTION)."""
+    heads: int
+    dim: int
+    vdim: int
+    decay: tuple
+    k_scale: float
+    rot: Rotation = None
+
+    def weight_shapes(self, p, W):
+        return {p + 'q': (self.heads * self.dim, W), p + 'k': (self.heads * self.dim, W), p + 'v': (self.heads * self.vdim, W), p + 'g': (self.heads * self.vdim, W),
+                p + 'o': (W, self.heads * self.vdim)}
+
+
+@dataclass(frozen=True)
+class ParallelMixer:
+    """Attention and retention on the same input, outputs added: left_scale * left + right_scale * right."""
+    left: HeadsMixer
+    right: RetentionMixer
+    left_scale: float = 1.0
+    right_scale: float = 1.0
+
+    def weight_shapes(self, p, W):
+        return {**self.left.weight_shapes(p + 'left.', W), **self.right.weight_shapes(p + 'right.', W)}
+
 
 @dataclass(frozen=True)
 class ExpertMixture:
@@ -148,11 +205,27 @@ class ExpertMixture:
     groups: int = 1
     keep: int = 1
 
+    def weight_shapes(self, p, W):
+        out = {p + 'router': (self.experts, W), p + 'correction': (self.experts,)}
+        for e in range(self.experts):
+            out.update({f'{p}e{e}.gate': (self.ff, W), f'{p}e{e}.up': (self.ff, W), f'{p}e{e}.down': (W, self.ff)})
+        return out
+
+
+@dataclass(frozen=True)
+class DenseFF:
+    """W_down act(W_up h) (CR_FF_DENSE)."""
+    ff: int
+    act: str = 'relu2'
+
+    def weight_shapes(self, p, W):
+        return {p + 'up': (self.ff, W), p + 'down': (W, self.ff)}
+
 
 @dataclass(frozen=True)
 class DecoderLayer:
-    mixer: LatentMixer
-    ff: ExpertMixture = None
+    mixer: object                    # LatentMixer, HeadsMixer, RetentionMixer or ParallelMixer
+    ff: object = None                # ExpertMixture, DenseFF or none
 
 
 @dataclass(frozen=True)
@@ -165,6 +238,11 @@ class DecoderSpec:
     loop: tuple = None               # (start, stop, times): layers [start, stop) run `times` times in a row
     softcap: float = 0.0             # 0: no cap on the logits
     sinusoid_base: float = 0.0       # > 0: a sinusoidal position vector is added to the embedding
+    norm_plain: bool = False         # the model's norms multiply by their weight (otherwise by one plus their weight)
+    post_norm: bool = True           # a sublayer's output goes through a norm of its own before it joins the residual
+    tied_head: bool = False          # logits from the embedding table
+    loop_in: bool = False            # x <- W [x; embedding] ahead of every pass of the looped span
+    side_dim: int = 0                # > 0: per-layer token input of this width after the feed-forward
 
     @property
     def passes(self):
@@ -177,17 +255,24 @@ class DecoderSpec:
 
     def weight_shapes(self):
         """name -> shape of every checkpoint tensor."""
-        W, out = self.width, {'embed': (self.vocab, self.width), 'final.norm': (self.width,), 'head': (self.vocab, self.width)}
+        W, out = self.width, {'embed': (self.vocab, self.width), 'final.norm': (self.width,)}
+        if not self.tied_head:
+            out['head'] = (self.vocab, W)
+        if self.loop_in and self.loop:
+            out['loop.in'] = (W, 2 * W)
+        if self.side_dim:
+            out['side.embed'] = (self.vocab, len(self.layers) * self.side_dim)
         for i, layer in enumerate(self.layers):
-            p, m = f'l{i}.', layer.mixer
-            out.update({p + 'norm1': (W,), p + 'norm1b': (W,), p + 'mix.dq': (m.q_rank, W), p + 'mix.dq.norm': (m.q_rank,), p + 'mix.uq': (m.heads * m.dim, m.q_rank),
-                        p + 'mix.dkv': (m.kv_rank, W), p + 'mix.dkv.norm': (m.kv_rank,), p + 'mix.uk': (m.heads * m.dim, m.kv_rank),
-                        p + 'mix.uv': (m.heads * m.vdim, m.kv_rank), p + 'mix.g': (m.heads * m.vdim, W), p + 'mix.o': (W, m.heads * m.vdim)})
-            if layer.ff is not None:
-                f = layer.ff
-                out.update({p + 'norm2': (W,), p + 'norm2b': (W,), p + 'mlp.router': (f.experts, W), p + 'mlp.correction': (f.experts,)})
-                for e in range(f.experts):
-                    out.update({f'{p}mlp.e{e}.gate': (f.ff, W), f'{p}mlp.e{e}.up': (f.ff, W), f'{p}mlp.e{e}.down': (W, f.ff)})
+            p = f'l{i}.'
+            for j, sub in enumerate((layer.mixer, layer.ff), 1):
+                if sub is None:
+                    continue
+                out[f'{p}norm{j}'] = (W,)
+                if self.post_norm:
+                    out[f'{p}norm{j}b'] = (W,)
+                out.update(sub.weight_shapes(p + ('mix.' if j == 1 else 'mlp.'), W))
+            if self.side_dim:
+                out.update({p + 'side.gate': (self.side_dim, W), p + 'side.proj': (W, self.side_dim), p + 'side.norm': (W,)})
         return out
 
     @staticmethod
@@ -209,3 +294,28 @@ class DecoderSpec:
         lp = cfg.get('loop')
         return DecoderSpec(width=cfg['width'], vocab=cfg['vocab'], layers=tuple(layers), eps=float(cfg['norm']['eps']),
                            loop=(lp['start'], lp['stop'], lp['times']) if lp else None, softcap=float(cfg.get('logit_softcap') or 0.0), sinusoid_base=10000.0)
+
+    @staticmethod
+    def from_lugasun(cfg):
+        """The Lugasun design's config.json (parsed)."""
+        def rotation(m):
+            r = m.get('rot')
+            return Rotation(base=float(r['base']), dims=r['dims']) if r and r['dims'] else None
+        layers = []
+        for i, entry in enumerate(cfg['layers']):
+            if entry['type'] != 'parallel':
+                raise ValueError(f'layer {i}: unknown mixer {entry["type"]!r}')
+            m = entry['mixer']
+            a, r = m['left'], m['right']
+            left = HeadsMixer(heads=a['heads'], kv_heads=a['kv_heads'], dim=a['dim'], vdim=a['vdim'], scale=float(a['scale']), rot=rotation(a),
+                              chunk=(a.get('mask') or {}).get('size') or 0, softcap=float(a.get('softcap') or 0.0), qk_norm=True)
+            if len(r['decay']) != r['heads']:
+                raise ValueError(f'layer {i}: {len(r["decay"])} decays for {r["heads"]} heads')
+            right = RetentionMixer(heads=r['heads'], dim=r['dim'], vdim=r['vdim'], decay=tuple(float(d) for d in r['decay']), k_scale=r['dim'] ** -0.5, rot=rotation(r))
+            mlp = entry.get('mlp')
+            if mlp is not None and mlp['kind'] != 'dense':
+                raise ValueError(f'layer {i}: unknown feed-forward {mlp["kind"]!r}')
+            layers.append(DecoderLayer(ParallelMixer(left, right, float(m['left_scale']), float(m['right_scale'])), DenseFF(mlp['ff']) if mlp is not None else None))
+        lp, side = cfg.get('loop'), cfg.get('token_side')
+        return DecoderSpec(width=cfg['width'], vocab=cfg['vocab'], layers=tuple(layers), eps=float(cfg['norm']['eps']), loop=(lp['start'], lp['stop'], lp['times']) if lp else None,
+                           norm_plain=True, post_norm=False, tied_head=True, loop_in=bool(lp), side_dim=side['dim'] if side else 0)

@@ -73,7 +73,8 @@ template <int D> __device__ __forceinline__ int vswz(int r) { return D == 64 ? (
 // 10 waves per CU: 0.62 ms) and of 8 waves (256 queries; one workgroup per CU: 0.56 ms) against 0.50-0.51 for these 4.  The lean tile is 138 vector instructions + 16 MFMAs +
 // 24 LDS reads per wave; per SIMD the three waves' vector (~1 340 cycles) and matrix (1 536) work would fit 2 880 cycles even
 // with no overlap at all, the measured round is ~5 400: the SIMD idles while all three waves sit at their workgroups' barriers.
-template <int D, bool CAUSAL, bool SPLIT = false, bool DIV = false, bool WIDE = false>
+// WIDE: 1 = 32-bit scores (attention.hpp: wide), 2 = and soft-capped
+template <int D, bool CAUSAL, bool SPLIT = false, bool DIV = false, int WIDE = 0>
 __global__ __launch_bounds__(256, D == 256 ? 1 : 2) void flash_attn_kernel(const AttnParams p) {
     extern __shared__ __attribute__((aligned(16))) char smem[];
     constexpr int ROWB = D * 2;
@@ -108,7 +109,7 @@ __global__ __launch_bounds__(256, D == 256 ? 1 : 2) void flash_attn_kernel(const
     const int split = SPLIT ? bx : 0;
     const int kvh = head / p.kv_group;
     int slot = p.seq_map ? p.seq_map[batch] : batch;
-    int Sk = p.sk_arr ? p.sk_arr[slot] + p.sk_add : p.Sk;
+    int Sk = p.sk_arr ? ((WIDE && p.sk_mod > 0) ? p.sk_arr[slot] % p.sk_mod : p.sk_arr[slot]) + p.sk_add : p.Sk;
     int Sq = p.Sq, q_pos0 = p.q_pos0;
     int64_t q_base = (int64_t)batch * p.q_bs, o_base = (int64_t)batch * p.o_bs;
     if (CAUSAL && p.seg) {                                    // several pages' prompts in one launch (wave-uniform)
@@ -177,7 +178,9 @@ __global__ __launch_bounds__(256, D == 256 ? 1 : 2) void flash_attn_kernel(const
         nt = min(nt, kmax / 64 + 1);
     }
     const int qpos = q_pos0 + qi_c;
-    const float sc2 = WIDE ? p.s_mul * LOG2E : LOG2E;
+    const float sc2 = WIDE == 1 ? p.s_mul * LOG2E : LOG2E;
+    // softcap * tanh(z / softcap) = softcap - 2 softcap / (1 + exp(2 z / softcap))
+    const float cap = p.softcap, cap2 = -2.0f * p.softcap, capx = WIDE == 2 ? 2.0f * LOG2E * p.s_mul / p.softcap : 0.f;
     const float inv_div = 1.0f / p.s_div;     // reference divides by sqrt(d); x * (1/d) differs from x / d by <= 1 fp32 ulp before the bf16 rounding
     int t_begin = 0;
     if (SPLIT) {
@@ -267,6 +270,10 @@ __global__ __launch_bounds__(256, D == 256 ? 1 : 2) void flash_attn_kernel(const
 #pragma unroll
                 for (int e = 0; e < 16; e += 2) {
                     float s0 = sacc[kb][e], s1 = sacc[kb][e + 1];
+                    if (WIDE == 2) {
+                        s0 = fmaf(cap2, __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(s0 * capx)), cap);
+                        s1 = fmaf(cap2, __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(s1 * capx)), cap);
+                    }
                     if (decltype(masked)::value) {
                         const int key = kt * 64 + kb * 32 + (e & 3) + 8 * (e >> 2) + 4 * hh;
                         s0 = (key < Sk && (!CAUSAL || key <= qpos)) ? s0 : -INFINITY;
@@ -280,7 +287,7 @@ __global__ __launch_bounds__(256, D == 256 ? 1 : 2) void flash_attn_kernel(const
                 }
         };
         if (need_mask) score_pass(std::true_type{}); else score_pass(std::false_type{});   // wave-uniform
-        float mloc = WIDE ? mraw * p.s_mul : lo_bf16(pack_bf16(mraw, mraw));
+        float mloc = WIDE == 2 ? mraw : WIDE ? mraw * p.s_mul : lo_bf16(pack_bf16(mraw, mraw));
         if (DIV) mloc = lo_bf16(pack_bf16(mloc * inv_div, mloc * inv_div));
         mloc = fmaxf(mloc, __shfl_xor(mloc, 32, 64));
         // deferred rescale: while no row's maximum grows by more than 8 the reference point m_run stays (P <= e^8 keeps
@@ -355,7 +362,7 @@ __global__ __launch_bounds__(256, D == 256 ? 1 : 2) void flash_attn_kernel(const
         }
         return;
     }
-    const float inv = 1.0f / l_tot;
+    const float inv = (WIDE && p.out_mul != 0.f ? p.out_mul : 1.0f) / l_tot;
     if (WIDE) {
         if (qi >= Sq) return;
         bf16* op = p.O + o_base + (int64_t)qi * p.o_rs + (int64_t)head * p.o_hs + 4 * hh;
@@ -408,13 +415,17 @@ int launch_d(const AttnParams& p, hipStream_t stream) {
     return hipGetLastError() == hipSuccess ? CR_OK : CR_ERR_HIP;
 }
 
-template <int D>
+template <int D, bool CAUSAL, bool SPLIT, int WIDE>
 int launch_wide(const AttnParams& p, hipStream_t stream) {
     constexpr int LDS = 2 * 2 * 64 * D * 2;
     static std::atomic<uint64_t> attr_done{0};
-    if (!cr_dyn_lds_once(attr_done, (const void*)flash_attn_kernel<D, true, false, false, true>, LDS)) return CR_ERR_HIP;
-    hipLaunchKernelGGL((flash_attn_kernel<D, true, false, false, true>), dim3((p.Sq + 127) / 128, p.H, p.B), dim3(256), LDS, stream, p);
+    if (!cr_dyn_lds_once(attr_done, (const void*)flash_attn_kernel<D, CAUSAL, SPLIT, false, WIDE>, LDS)) return CR_ERR_HIP;
+    hipLaunchKernelGGL((flash_attn_kernel<D, CAUSAL, SPLIT, false, WIDE>), dim3(SPLIT ? p.nsplit : (p.Sq + 127) / 128, p.H, p.B), dim3(256), LDS, stream, p);
     return hipGetLastError() == hipSuccess ? CR_OK : CR_ERR_HIP;
+}
+template <int D>
+int launch_wide(const AttnParams& p, hipStream_t stream) {
+    return p.softcap > 0.f ? launch_wide<D, true, false, 2>(p, stream) : launch_wide<D, true, false, 1>(p, stream);
 }
 
 template <int D, bool CAUSAL>
@@ -454,7 +465,8 @@ __global__ __launch_bounds__(D) void attn_combine_kernel(const AttnParams p) {
             }
         }
     }
-    p.O[(int64_t)batch * p.o_bs + (int64_t)q * p.o_rs + (int64_t)head * p.o_hs + d] = f2bf(acc / L);
+    if (p.wide && d >= p.vdim) return;
+    p.O[(int64_t)batch * p.o_bs + (int64_t)q * p.o_rs + (int64_t)head * p.o_hs + d] = f2bf(p.wide && p.out_mul != 0.f ? p.out_mul * acc / L : acc / L);
 }
 
 template <int D, bool DIV>
@@ -463,6 +475,14 @@ int launch_split_d(const AttnParams& p, hipStream_t stream) {
     static std::atomic<uint64_t> attr_done{0};
     if (!cr_dyn_lds_once(attr_done, (const void*)flash_attn_kernel<D, false, true, DIV>, LDS)) return CR_ERR_HIP;
     hipLaunchKernelGGL((flash_attn_kernel<D, false, true, DIV>), dim3(p.nsplit, p.H, p.B), dim3(256), LDS, stream, p);
+    hipLaunchKernelGGL((attn_combine_kernel<D>), dim3(p.Sq, p.H, p.B), dim3(D), 0, stream, p);
+    return hipGetLastError() == hipSuccess ? CR_OK : CR_ERR_HIP;
+}
+
+template <int D>
+int launch_split_wide(const AttnParams& p, hipStream_t stream) {
+    const int rc = p.softcap > 0.f ? launch_wide<D, false, true, 2>(p, stream) : launch_wide<D, false, true, 1>(p, stream);
+    if (rc != CR_OK) return rc;
     hipLaunchKernelGGL((attn_combine_kernel<D>), dim3(p.Sq, p.H, p.B), dim3(D), 0, stream, p);
     return hipGetLastError() == hipSuccess ? CR_OK : CR_ERR_HIP;
 }
@@ -477,6 +497,13 @@ int launch_flash_attn_split(const AttnParams& p, int head_dim, hipStream_t strea
     if (p.Sq <= 0 || p.Sq > 32 || p.H <= 0 || p.B <= 0 || p.nsplit <= 0 || !p.part_ml || !p.part_o) return CR_ERR_ARG;
     if ((p.q_rs & 7) || (p.k_rs & 7) || (p.v_rs & 7)) return CR_ERR_ARG;
     const bool dv = p.s_div != 1.0f;
+    if (p.wide) {
+        if (p.s_mul <= 0.f || p.vdim <= 0 || p.vdim > head_dim || p.q_prescale != 1.f || dv || p.gate) return CR_ERR_ARG;
+        if (head_dim == 64) return launch_split_wide<64>(p, stream);
+        if (head_dim == 128) return launch_split_wide<128>(p, stream);
+        if (head_dim == 256) return launch_split_wide<256>(p, stream);
+        return CR_ERR_ARG;
+    }
     if (decode_attn_supported(p, head_dim)) {                 // attention_decode.hip writes the same partials; the combine is this file's
         if (launch_decode_attn(p, stream) != CR_OK) return CR_ERR_HIP;
         hipLaunchKernelGGL((attn_combine_kernel<128>), dim3(p.Sq, p.H, p.B), dim3(128), 0, stream, p);

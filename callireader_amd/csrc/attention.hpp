@@ -36,8 +36,11 @@ struct AttnParams {
     const bf16* rope_sin;
     // 32-bit scores (causal prefill only): score = (q . k) * s_mul in fp32 with no rounding before the softmax, the fp32 weights enter P.V as the sum of two bf16 halves;
     // head h's `vdim` output columns start at column h * o_hs, each multiplied by sigmoid(gate[row][h * vdim + d]) when `gate` is given (rows g_rs apart)
+    // (decode: launch_flash_attn_split with `wide`, no gate).  softcap > 0: the score becomes softcap * tanh(score / softcap); out_mul (0 = 1) multiplies the result
     int wide;
     float s_mul;              // > 0
+    float softcap, out_mul;
+    int sk_mod;               // decode: > 0: a row sees the last sk_arr[slot] % sk_mod + sk_add keys, which start at its slot's first row
     int vdim;
     const bf16* gate; int64_t g_rs;
 };

@@ -123,6 +123,13 @@ __device__ __forceinline__ void store16_e4m3(unsigned char* dst, const float* y,
     *(u32x4_*)dst = w;
 }
 
+// max(x, 0)^2
+__device__ __forceinline__ float relu2(float x) { const float r = fmaxf(x, 0.f); return r * r; }
+// 0.5 x (1 + tanh(sqrt(2 / pi) (x + 0.044715 x^3))) = x / (1 + exp(-2 t))
+__device__ __forceinline__ float gelu_tanh(float x) {
+    const float t = 0.7978845608028654f * (x + 0.044715f * x * x * x);
+    return x / (1.0f + expf(-2.0f * t));
+}
 __device__ __forceinline__ float silu(float x) { return x / (1.0f + __expf(-x)); }
 
 __device__ __forceinline__ float wave_sum(float v) {
@@ -163,6 +170,7 @@ enum GemmEpi {
     EPI_GELU_Q8 = 9,  // e4m3 instance only: e4m3(bf16(gelu(bf16(acc + bias))) / c8scale[m]) -- fc1's output as fc2's fp8 operand, no bf16 copy
     EPI_X_GLU = 10,   // grouped experts (gemm256 only): rows gathered through `perm`, W rows interleaved [8 gate | 8 up], clamped gated unit (GemmParams::limit)
     EPI_X_ROWS = 11,  // grouped experts (gemm256 only): plain rows, scattered through `perm`
+    EPI_RELU2 = 12,   // bf16(max(acc, 0)^2), no bias
     EPI_ARGMAX = 8,   // cosine VQ: C[m][b] = {col, bits(max)} of bf16(acc) over the 64 columns of block b (first max wins); nothing else stored
 };
 

@@ -164,6 +164,10 @@ __device__ __forceinline__ void stage_slice(const f32x4 (&a)[4], const float (&b
         }
 #pragma unroll
         for (int e = 0; e < 4; e++) x[e] += bias_f[j][e];               // -0.0f where there is no bias: x + -0 = x, bit for bit
+        if (EPI == EPI_RELU2) {
+#pragma unroll
+            for (int e = 0; e < 4; e++) x[e] = relu2(x[e]);
+        }
         if (EPI == EPI_GELU || EPI == EPI_LS_RES) {          // bf16(acc + bias) is a value of its own before the next op
             round_pair_bf16(x[0], x[1], x[0], x[1]);
             round_pair_bf16(x[2], x[3], x[2], x[3]);
@@ -897,6 +901,7 @@ int launch_gemm256(int epi, const GemmParams& p, hipStream_t stream) {
     switch (epi) {
         case EPI_STORE: return launch_t<EPI_STORE>(p, stream);
         case EPI_GELU: return launch_t<EPI_GELU>(p, stream);
+        case EPI_RELU2: return launch_t<EPI_RELU2>(p, stream);
         case EPI_LS_RES: return launch_t<EPI_LS_RES>(p, stream);
         case EPI_RES: return launch_t<EPI_RES>(p, stream);
         case EPI_SWIGLU: return launch_t<EPI_SWIGLU>(p, stream);

@@ -246,7 +246,7 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_skinny_kernel(const GemmParam
         if (gm >= p.M || gn >= p.N) continue;
         const float sum = red[0][t][n][m] + (p.bias ? bf2f(p.bias[gn]) : 0.f);
         if (EPI == EPI_F32) { ((float*)p.C)[(int64_t)gm * p.ldc + gn] = f32_out(p, sum); continue; }
-        float x = rbf(sum);
+        float x = EPI == EPI_RELU2 ? relu2(sum) : rbf(sum);
         if (EPI == EPI_GELU) x = gelu_erf(x);
         if (EPI == EPI_LS_RES) x = bf2f(p.res[(int64_t)gm * p.ldr + gn]) + rbf(x * bf2f(p.scale[gn]));
         if (EPI == EPI_RES) x = bf2f(p.res[(int64_t)gm * p.ldr + gn]) + x;
@@ -331,13 +331,14 @@ bool gemm_tail_supported(int epi, const GemmParams& p) {
     if (epi == EPI_LS_RES) return p.res && p.scale;
     if (epi == EPI_RES) return p.res != nullptr;
     if (epi == EPI_SWIGLU) return p.N % 16 == 0;
-    return epi == EPI_STORE || epi == EPI_GELU || epi == EPI_F32;
+    return epi == EPI_STORE || epi == EPI_GELU || epi == EPI_RELU2 || epi == EPI_F32;
 }
 
 int launch_gemm_tail(int epi, const GemmParams& p, hipStream_t stream) {
     switch (epi) {
         case EPI_STORE: return launch_mt8<EPI_STORE, 1, 1, false>(p, stream, 1);
         case EPI_GELU: return launch_mt8<EPI_GELU, 1, 1, false>(p, stream, 1);
+        case EPI_RELU2: return launch_mt8<EPI_RELU2, 1, 1, false>(p, stream, 1);
         case EPI_LS_RES: return launch_mt8<EPI_LS_RES, 1, 1, false>(p, stream, 1);
         case EPI_RES: return launch_mt8<EPI_RES, 1, 1, false>(p, stream, 1);
         case EPI_SWIGLU: return launch_mt8<EPI_SWIGLU, 1, 1, false>(p, stream, 1);
@@ -353,6 +354,7 @@ bool gemm_skinny_supported(int epi, const GemmParams& p) {
     if (p.w8 && (p.K % 512 != 0 || !p.wscale || (p.ldw & 15))) return false;
     if (epi == EPI_PARTIAL) return p.bias == nullptr && partial_geom(p.N, p.K).splits > 0;
     if (epi == EPI_STORE || epi == EPI_F32) return true;
+    if (epi == EPI_RELU2) return !p.w8;
     if (epi == EPI_RES) return p.res != nullptr;
     if (epi == EPI_SWIGLU) return p.N % 16 == 0;
     return false;
@@ -366,6 +368,7 @@ int launch_gemm_skinny(int epi, const GemmParams& p, hipStream_t stream) {
         case EPI_RES: return launch_w<EPI_RES>(p, stream);
         case EPI_SWIGLU: return launch_w<EPI_SWIGLU>(p, stream);
         case EPI_F32: return launch_w<EPI_F32>(p, stream);
+        case EPI_RELU2: return launch_w<EPI_RELU2>(p, stream);
         case EPI_PARTIAL: {
             const PartialGeom g = partial_geom(p.N, p.K);
             switch (g.rt) {

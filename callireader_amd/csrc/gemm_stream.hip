@@ -186,7 +186,7 @@ __global__ __launch_bounds__(NW * 64) void gemm_stream_kernel(const GemmParams p
         for (int e = 0; e < 4; e++) {
             if (gn + e >= p.N) continue;
             if (EPI == EPI_F32) { ((float*)p.C)[(int64_t)gm * p.ldc + gn + e] = f32_out(p, acc[t][e] + bias[e]); continue; }
-            float x = rbf(acc[t][e] + bias[e]);
+            float x = EPI == EPI_RELU2 ? relu2(acc[t][e] + bias[e]) : rbf(acc[t][e] + bias[e]);
             if (EPI == EPI_RES) x = bf2f(p.res[(int64_t)gm * p.ldr + gn + e]) + x;
             ((bf16*)p.C)[(int64_t)gm * p.ldc + gn + e] = f2bf(x);
         }
@@ -263,7 +263,7 @@ bool gemm_stream_supported(int epi, const GemmParams& p, int splits) {
     if (p.a8 || p.M <= min_rows || p.M > 64 || splits != 1 || p.N <= 8192 || p.K % 2048 != 0 || p.wsw > 1) return false;
     if (p.w8 && ((epi != EPI_SWIGLU && epi != EPI_F32) || !p.wscale || (!p.wsw && (p.ldw & 15)) || p.bias)) return false;      // e4m3 weights: the two shapes decode streams here
     if ((p.lda & 7) || (!p.wsw && (p.ldw & 7)) || ((uintptr_t)p.A & 15) || ((uintptr_t)p.W & 15)) return false;
-    if (epi == EPI_STORE || epi == EPI_F32) return true;
+    if (epi == EPI_STORE || epi == EPI_F32 || epi == EPI_RELU2) return true;
     if (epi == EPI_RES) return p.res != nullptr;
     if (epi == EPI_SWIGLU) return p.N % 16 == 0 && (p.ldc & 3) == 0 && ((uintptr_t)p.C & 7) == 0;
     return false;
@@ -276,6 +276,7 @@ int launch_gemm_stream(int epi, const GemmParams& p, hipStream_t stream, int spl
         case EPI_RES: return launch_e<EPI_RES>(p, stream, splits, nw);
         case EPI_SWIGLU: return launch_e<EPI_SWIGLU>(p, stream, splits, nw);
         case EPI_F32: return launch_e<EPI_F32>(p, stream, splits, nw);
+        case EPI_RELU2: return launch_e<EPI_RELU2>(p, stream, splits, nw);
     }
     return CR_ERR_ARG;
 }

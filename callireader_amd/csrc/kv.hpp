@@ -10,8 +10,10 @@ struct cr_kv {
     int n_seqs, max_tokens, gen_cap, layers;
     bf16* k;             // [layers][n_seqs][8][max_tokens][128]
     bf16* v;
-    char* lat;           // described decoders: layer pass r at lat + lat_off[r] bytes: [n_seqs][max_tokens][padded kv_rank] in the model's element type
-    std::vector<size_t> lat_off;
+    // described decoders: what layer pass r keeps starts at lat + lat_off[r] bytes: latent rows [n_seqs][max_tokens][padded kv_rank] in the model's element type, or keys and values
+    // [2][n_seqs][kv_heads][ring][padded head] (ring = the rows a chunk needs); retention's fp32 states [n_seqs][heads][..] at lat + state_off[r]
+    char* lat;
+    std::vector<size_t> lat_off, state_off;
     int32_t* d_len;      // [n_seqs] tokens cached
     int32_t* d_ngen;     // [n_seqs] ids generated
     int64_t* d_gen;      // [n_seqs][gen_cap]

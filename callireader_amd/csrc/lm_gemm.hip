@@ -127,6 +127,15 @@ __global__ __launch_bounds__(256) void lm_gemm_kernel(const LmGemmParams p) {
 #pragma unroll
                 for (int e = 0; e < 4; e++)
                     if (n + e < p.N) c[e] = (T)(v[e] / (1.0f + expf(-(float)g[e])));
+            } else if (EPI == LM_SIDE) {
+                const T* g = (const T*)p.gate + (int64_t)p.tok[cr] * p.ldg + n;
+#pragma unroll
+                for (int e = 0; e < 4; e++)
+                    if (n + e < p.N) c[e] = (T)(gelu_tanh(v[e]) * (float)g[e]);
+            } else if (EPI == LM_RELU2) {
+#pragma unroll
+                for (int e = 0; e < 4; e++)
+                    if (n + e < p.N) c[e] = (T)relu2(v[e]);
             } else {
 #pragma unroll
                 for (int e = 0; e < 4; e++)
@@ -144,6 +153,8 @@ int launch_t(int epi, const LmGemmParams& p, hipStream_t st) {
         case LM_RAW32: hipLaunchKernelGGL((lm_gemm_kernel<T, LM_RAW32>), grid, block, 0, st, p); break;
         case LM_GLU: hipLaunchKernelGGL((lm_gemm_kernel<T, LM_GLU>), grid, block, 0, st, p); break;
         case LM_GATE: hipLaunchKernelGGL((lm_gemm_kernel<T, LM_GATE>), grid, block, 0, st, p); break;
+        case LM_RELU2: hipLaunchKernelGGL((lm_gemm_kernel<T, LM_RELU2>), grid, block, 0, st, p); break;
+        case LM_SIDE: hipLaunchKernelGGL((lm_gemm_kernel<T, LM_SIDE>), grid, block, 0, st, p); break;
         default: return cr_fail(CR_ERR_ARG, "lm_gemm: epilogue %d", epi);
     }
     CR_HIP(hipGetLastError());
@@ -155,7 +166,7 @@ int launch_t(int epi, const LmGemmParams& p, hipStream_t st) {
 int launch_lm_gemm(bool f32, int epi, const LmGemmParams& p, hipStream_t st) {
     const int vec = f32 ? 4 : 8;
     if (p.N <= 0 || p.K <= 0 || p.K % 64 || p.lda % vec || p.ldw % vec || p.a_bs % vec || p.w_bs % vec || (p.tiles ? p.max_tiles <= 0 || p.batch > 1 || !p.n_tiles : p.M <= 0) ||
-        (p.gather_div && !p.perm) || (epi == LM_GLU && (p.N % 16 || p.batch > 1)) || (epi == LM_GATE && !p.gate) || (((uintptr_t)p.A | (uintptr_t)p.W) & 15))
+        (p.gather_div && !p.perm) || (epi == LM_GLU && (p.N % 16 || p.batch > 1)) || ((epi == LM_GATE || epi == LM_SIDE) && !p.gate) || (epi == LM_SIDE && !p.tok) || (((uintptr_t)p.A | (uintptr_t)p.W) & 15))
         return cr_fail(CR_ERR_ARG, "lm_gemm(epi=%d M=%d N=%d K=%d): bad argument", epi, p.M, p.N, p.K);
     return f32 ? launch_t<float>(epi, p, st) : launch_t<bf16>(epi, p, st);
 }

@@ -45,19 +45,33 @@ __device__ __forceinline__ void norm_store(const f32x4 (&x)[NV], int Wp, int W, 
     }
 }
 
+// the row for its next reader: rms(x) * gain, or x itself
+template <typename T, int TPB, int NV>
+__device__ __forceinline__ void sink_store(const f32x4 (&x)[NV], int Wp, int W, float eps, const LmSink& to, int64_t row, float* red, int tid) {
+    if (!to.h) return;
+    T* h = (T*)to.h + row * to.ldh;
+    if (to.gain) { norm_store<T, TPB, NV>(x, Wp, W, eps, to.gain, h, red, tid); return; }
+#pragma unroll
+    for (int j = 0; j < NV; j++) {
+        const int i = 4 * tid + 4 * TPB * j;
+        if (i < Wp) st4(h + i, x[j]);
+    }
+}
+
 __device__ __forceinline__ int row_seq(const LmRowIndex& ix, int row) { return ix.row_seq ? ix.row_seq[row] : ix.seqs[row]; }
 __device__ __forceinline__ int row_pos(const LmRowIndex& ix, int row) { return ix.row_pos ? ix.row_pos[row] : ix.lens[ix.seqs[row]]; }
 
 template <typename T, int TPB, int NV>
 __global__ __launch_bounds__(TPB) void lm_embed_kernel(const T* __restrict__ table, const float* __restrict__ freq, int Wp, int W, int vocab, float eps, const int64_t* __restrict__ tokens,
                                                        const LmRowIndex ix, const int64_t* __restrict__ gen, const int32_t* __restrict__ ngen, int gen_cap,
-                                                       float* __restrict__ xo, T* __restrict__ h, const float* __restrict__ gain) {
+                                                       float* __restrict__ xo, const LmSink to, int32_t* __restrict__ tok, T* __restrict__ x0, int64_t ldx0) {
     __shared__ float red[TPB / 64];
     const int row = blockIdx.x, tid = threadIdx.x;
     const int seq = row_seq(ix, row);
     const float pos = (float)row_pos(ix, row);
     const int64_t t = tokens ? tokens[row] : gen[(int64_t)seq * gen_cap + ngen[seq] - 1];
     const int64_t id = t < 0 ? 0 : (t >= vocab ? vocab - 1 : t);      // (the host checks ids; a clamped read stays in bounds whatever arrives)
+    if (tok && tid == 0) tok[row] = (int32_t)id;
     f32x4 x[NV];
 #pragma unroll
     for (int j = 0; j < NV; j++) {
@@ -72,13 +86,14 @@ __global__ __launch_bounds__(TPB) void lm_embed_kernel(const T* __restrict__ tab
             x[j][q] = e[q] + s;
         }
         *(f32x4*)(xo + (int64_t)row * Wp + i) = x[j];
+        if (x0) st4(x0 + (int64_t)row * ldx0 + i, x[j]);
     }
-    norm_store<T, TPB, NV>(x, Wp, W, eps, gain, h + (int64_t)row * Wp, red, tid);
+    sink_store<T, TPB, NV>(x, Wp, W, eps, to, row, red, tid);
 }
 
 template <typename T, int TPB, int NV>
 __global__ __launch_bounds__(TPB) void lm_post_kernel(const LmPostIn in, int M, int Wp, int W, float eps, float* __restrict__ xio,
-                                                      const float* __restrict__ gain_b, T* __restrict__ h, const float* __restrict__ gain_next) {
+                                                      const float* __restrict__ gain_b, int replace, const LmSink to) {
     __shared__ float red[TPB / 64];
     const int tid = threadIdx.x;
     const int64_t row = blockIdx.x;
@@ -88,7 +103,7 @@ __global__ __launch_bounds__(TPB) void lm_post_kernel(const LmPostIn in, int M, 
         const int i = 4 * tid + 4 * TPB * j;
         x[j] = y[j] = f32x4{0.f, 0.f, 0.f, 0.f};
         if (i >= Wp) continue;
-        x[j] = *(const f32x4*)(xio + row * Wp + i);
+        if (!replace) x[j] = *(const f32x4*)(xio + row * Wp + i);
         if (in.slices) {                                       // K-slices of a weight-streaming product, in slice order
             for (int k = 0; k < in.slices; k += 4) {
                 f32x4 v[4];
@@ -113,18 +128,21 @@ __global__ __launch_bounds__(TPB) void lm_post_kernel(const LmPostIn in, int M, 
                     if (k + q < in.top) y[j] += w[q] * v[q];
             }
     }
-    float ss = 0.f;
+    float rs = 1.f;
+    if (gain_b) {
+        float ss = 0.f;
 #pragma unroll
-    for (int j = 0; j < NV; j++) ss += sumsq4(y[j]);
-    const float rs = 1.0f / sqrtf(block_sum<TPB>(ss, red, tid) / (float)W + eps);
+        for (int j = 0; j < NV; j++) ss += sumsq4(y[j]);
+        rs = 1.0f / sqrtf(block_sum<TPB>(ss, red, tid) / (float)W + eps);
+    }
 #pragma unroll
     for (int j = 0; j < NV; j++) {
         const int i = 4 * tid + 4 * TPB * j;
         if (i >= Wp) continue;
-        x[j] += y[j] * rs * *(const f32x4*)(gain_b + i);
+        x[j] += gain_b ? y[j] * rs * *(const f32x4*)(gain_b + i) : y[j];
         *(f32x4*)(xio + row * Wp + i) = x[j];
     }
-    if (gain_next) norm_store<T, TPB, NV>(x, Wp, W, eps, gain_next, h + row * Wp, red, tid);
+    sink_store<T, TPB, NV>(x, Wp, W, eps, to, row, red, tid);
 }
 
 template <typename T, int TPB, int NV>
@@ -220,15 +238,15 @@ __global__ __launch_bounds__(256) void lm_latents_kernel(T* __restrict__ a, cons
         return CR_OK;                                                                                                 \
     } while (0)
 
-int launch_lm_embed(bool f32, const Lm& lm, int M, const int64_t* tokens, const LmRowIndex& ix, const int64_t* gen, const int32_t* ngen, int gen_cap, float* x, void* h, const float* gain,
-                    hipStream_t st) {
-    if (f32) LM_NV_DISPATCH(lm_embed_kernel, float, M, (const float*)lm.embed, lm.freq, lm.Wp, lm.d.width, lm.d.vocab, lm.d.eps, tokens, ix, gen, ngen, gen_cap, x, (float*)h, gain);
-    LM_NV_DISPATCH(lm_embed_kernel, bf16, M, (const bf16*)lm.embed, lm.freq, lm.Wp, lm.d.width, lm.d.vocab, lm.d.eps, tokens, ix, gen, ngen, gen_cap, x, (bf16*)h, gain);
+int launch_lm_embed(bool f32, const Lm& lm, int M, const int64_t* tokens, const LmRowIndex& ix, const int64_t* gen, const int32_t* ngen, int gen_cap, float* x, const LmSink& to, int32_t* tok,
+                    void* x0, int64_t ldx0, hipStream_t st) {
+    if (f32) LM_NV_DISPATCH(lm_embed_kernel, float, M, (const float*)lm.embed, lm.freq, lm.Wp, lm.d.width, lm.d.vocab, lm.d.eps, tokens, ix, gen, ngen, gen_cap, x, to, tok, (float*)x0, ldx0);
+    LM_NV_DISPATCH(lm_embed_kernel, bf16, M, (const bf16*)lm.embed, lm.freq, lm.Wp, lm.d.width, lm.d.vocab, lm.d.eps, tokens, ix, gen, ngen, gen_cap, x, to, tok, (bf16*)x0, ldx0);
 }
 
-int launch_lm_post(bool f32, const Lm& lm, int M, const LmPostIn& in, float* x, const float* gain_b, void* h, const float* gain_next, hipStream_t st) {
-    if (f32) LM_NV_DISPATCH(lm_post_kernel, float, M, in, M, lm.Wp, lm.d.width, lm.d.eps, x, gain_b, (float*)h, gain_next);
-    LM_NV_DISPATCH(lm_post_kernel, bf16, M, in, M, lm.Wp, lm.d.width, lm.d.eps, x, gain_b, (bf16*)h, gain_next);
+int launch_lm_post(bool f32, const Lm& lm, int M, const LmPostIn& in, float* x, const float* gain_b, bool replace, const LmSink& to, hipStream_t st) {
+    if (f32) LM_NV_DISPATCH(lm_post_kernel, float, M, in, M, lm.Wp, lm.d.width, lm.d.eps, x, gain_b, (int)replace, to);
+    LM_NV_DISPATCH(lm_post_kernel, bf16, M, in, M, lm.Wp, lm.d.width, lm.d.eps, x, gain_b, (int)replace, to);
 }
 
 int launch_lm_pick_rows(bool f32, const Lm& lm, int n, const float* x, const int32_t* rows, void* h, const float* gain, hipStream_t st) {
@@ -246,6 +264,26 @@ int launch_lm_latents(bool f32, const Lm& lm, const LmLayer& L, int M, void* a, 
     else
         hipLaunchKernelGGL(lm_latents_kernel<bf16>, grid, dim3(256), 0, st, (bf16*)a, part, slices, M, L.Na, L.s.q_rank, L.Qp, L.off_c, L.s.kv_rank, L.Rp, L.off_g, lm.d.eps, L.nq, L.nc,
                            (bf16*)cq, (bf16*)c_dense, (bf16*)cache, max_tokens, ix, (bf16*)ao, n_ao, L.Gp);
+    CR_HIP(hipGetLastError());
+    return CR_OK;
+}
+
+namespace {
+// z[m][n] = gelu_tanh(sum of K-slices) * side[tok[m]][n], one thread per four columns
+__global__ __launch_bounds__(256) void lm_side_act_kernel(const float* __restrict__ part, int slices, int M, int Sp, const bf16* __restrict__ side, int64_t lds, const int32_t* __restrict__ tok,
+                                                          bf16* __restrict__ z) {
+    const int i = (blockIdx.x * 256 + threadIdx.x) * 4;
+    if (i >= M * Sp) return;
+    const int m = i / Sp, n = i - m * Sp;
+    f32x4 s = {0.f, 0.f, 0.f, 0.f};
+    for (int k = 0; k < slices; k++) s += *(const f32x4*)(part + ((int64_t)k * M + m) * Sp + n);
+    const f32x4 e = ld4(side + (int64_t)tok[m] * lds + n);
+    st4(z + i, f32x4{gelu_tanh(s[0]) * e[0], gelu_tanh(s[1]) * e[1], gelu_tanh(s[2]) * e[2], gelu_tanh(s[3]) * e[3]});
+}
+}  // namespace
+
+int launch_lm_side_act(const Lm& lm, int M, const float* part, int slices, const void* side, int64_t lds, const int32_t* tok, void* z, hipStream_t st) {
+    hipLaunchKernelGGL(lm_side_act_kernel, dim3((M * lm.Sp / 4 + 255) / 256), dim3(256), 0, st, part, slices, M, lm.Sp, (const bf16*)side, lds, tok, (bf16*)z);
     CR_HIP(hipGetLastError());
     return CR_OK;
 }

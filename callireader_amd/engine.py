@@ -5,7 +5,7 @@ import ctypes as C
 import torch
 
 from . import _binding as B
-from .config import DecoderSpec, ModelDims
+from .config import DecoderSpec, DenseFF, HeadsMixer, ModelDims, ParallelMixer, RetentionMixer
 
 _DT = {torch.bfloat16: B.CR_BF16, torch.float32: B.CR_F32, torch.int64: B.CR_I64, torch.int32: B.CR_I32}
 
@@ -249,6 +249,23 @@ class Engine:
         return logits
 
 
+def _describe_mixer(c, m, name=b'', out_scale=1.0):
+    """Fill cr_lm_layer `c` with mixer `m`; two mixers side by side set both of its parts."""
+    if isinstance(m, ParallelMixer):
+        _describe_mixer(c, m.left, b'left.', m.left_scale)
+        _describe_mixer(c, m.right, b'right.', m.right_scale)
+    elif isinstance(m, HeadsMixer):
+        c.mixer |= B.CR_MIX_HEADS
+        c.attn = B.LmHeads(name=name, heads=m.heads, kv_heads=m.kv_heads, dim=m.dim, vdim=m.vdim, chunk=m.chunk, qk_norm=m.qk_norm, rot_dims=m.rot.dims if m.rot else 0,
+                           rot_base=m.rot.base if m.rot else 1.0, scale=m.scale, softcap=m.softcap, out_scale=out_scale)
+    elif isinstance(m, RetentionMixer):
+        c.mixer |= B.CR_MIX_RETENTION
+        c.ret = B.LmRetention(name=name, heads=m.heads, dim=m.dim, vdim=m.vdim, rot_dims=m.rot.dims if m.rot else 0, rot_base=m.rot.base if m.rot else 1.0, k_scale=m.k_scale,
+                              out_scale=out_scale, decay=(C.c_double * m.heads)(*m.decay))
+    else:
+        c.mixer, c.heads, c.dim, c.vdim, c.q_rank, c.kv_rank, c.scale = B.CR_MIX_LATENT, m.heads, m.dim, m.vdim, m.q_rank, m.kv_rank, m.scale
+
+
 class DecoderEngine(Engine):
     """A context whose language model is a described decoder (cr_lm_configure): token ids in, the same cache object, decode step and greedy pick."""
 
@@ -259,13 +276,16 @@ class DecoderEngine(Engine):
         self.spec, self.dtype = spec, dtype
         a, z, t = spec.loop or (0, 0, 0)
         d = B.LmDesc(layers=len(spec.layers), width=spec.width, vocab=spec.vocab, dtype=_DT[dtype], loop_start=a, loop_stop=z, loop_times=t,
-                     pos=B.CR_POS_SINUSOID if spec.sinusoid_base > 0 else B.CR_POS_NONE, pos_base=spec.sinusoid_base, eps=spec.eps, softcap=spec.softcap)
+                     pos=B.CR_POS_SINUSOID if spec.sinusoid_base > 0 else B.CR_POS_NONE, pos_base=spec.sinusoid_base, eps=spec.eps, softcap=spec.softcap, norm_plain=spec.norm_plain,
+                     no_post_norm=not spec.post_norm, tied_head=spec.tied_head, loop_in=spec.loop_in, side_dim=spec.side_dim)
         layers = (B.LmLayer * len(spec.layers))()
         for c, s in zip(layers, spec.layers):
-            m, f = s.mixer, s.ff
-            c.mixer, c.heads, c.dim, c.vdim, c.q_rank, c.kv_rank, c.scale = B.CR_MIX_LATENT, m.heads, m.dim, m.vdim, m.q_rank, m.kv_rank, m.scale
+            _describe_mixer(c, s.mixer)
+            f = s.ff
             c.ff = B.CR_FF_NONE
-            if f is not None:
+            if isinstance(f, DenseFF):
+                c.ff, c.expert_ff, c.act = B.CR_FF_DENSE, f.ff, {'relu2': B.CR_ACT_RELU2}[f.act]
+            elif f is not None:
                 c.ff, c.experts, c.top, c.expert_ff, c.groups, c.keep, c.limit = B.CR_FF_MOE, f.experts, f.top, f.ff, f.groups, f.keep, f.limit
         B.check(B.lib.cr_lm_configure(self._h, C.byref(d), layers), 'cr_lm_configure')
 

@@ -113,3 +113,8 @@ class DecoderLM:
 class LinasunForCausalLM(DecoderLM):
     """Looped latent-attention decoder with clamped expert mixtures, norms on both sides of every sublayer and soft-capped logits."""
     read_config = staticmethod(DecoderSpec.from_linasun)
+
+
+class LugasunForCausalLM(DecoderLM):
+    """Looped decoder whose layers run chunked attention and retention side by side, with a squared-relu feed-forward and a per-layer token input."""
+    read_config = staticmethod(DecoderSpec.from_lugasun)

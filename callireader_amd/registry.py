@@ -7,6 +7,7 @@ import os
 MODELS = {
     'InternVLChatModel': ('.modeling_internvl_chat', 'InternVLChatModel'),
     'Linasun': ('.modeling_decoder', 'LinasunForCausalLM'),
+    'Lugasun': ('.modeling_decoder', 'LugasunForCausalLM'),
 }
 DEFAULT = 'InternVLChatModel'            # the reference's checkpoints, and directories without a config.json
 

@@ -25,7 +25,7 @@
 extern "C" {
 #endif
 
-#define CR_ABI_VERSION 11  /* 11: cr_lm_configure, cr_lm_passes, cr_llm_prefill_tokens; 10: cr_op_decode_attention(+_scratch_floats); 9: cr_build_flags, cr_diag_register; 8: cr_op_decode_swizzle, cr_op_decode_gemm flags bit 8, cr_op_gemm bits 18-19; 7: cr_op_decode_gemm; 6: cr_build_id, cr_llm_hidden_probe; 5: cr_share_weights, cr_op_gemm_q8, cr_op_norm_fp8 takes the next linear's bound; 4: cr_enable_fp8_mfma, cr_op_norm_fp8, cr_op_gemm bit 17; 2: cr_orderformer; cr_op_gemm kernel pin and EPI_PARTIAL (epi 7); 3: cr_profile_stats, cr_kv_read, cr_kv_reset takes a stream, cr_enable_fp8_decode, cr_op_quantize_fp8, epi 8 */
+#define CR_ABI_VERSION 12  /* 12: cr_lm_layer / cr_lm_desc: attention over heads, retention, dense feed-forward, token side input; 11: cr_lm_configure, cr_lm_passes, cr_llm_prefill_tokens; 10: cr_op_decode_attention(+_scratch_floats); 9: cr_build_flags, cr_diag_register; 8: cr_op_decode_swizzle, cr_op_decode_gemm flags bit 8, cr_op_gemm bits 18-19; 7: cr_op_decode_gemm; 6: cr_build_id, cr_llm_hidden_probe; 5: cr_share_weights, cr_op_gemm_q8, cr_op_norm_fp8 takes the next linear's bound; 4: cr_enable_fp8_mfma, cr_op_norm_fp8, cr_op_gemm bit 17; 2: cr_orderformer; cr_op_gemm kernel pin and EPI_PARTIAL (epi 7); 3: cr_profile_stats, cr_kv_read, cr_kv_reset takes a stream, cr_enable_fp8_decode, cr_op_quantize_fp8, epi 8 */
 
 enum { CR_OK = 0, CR_ERR_ARG = -1, CR_ERR_HIP = -2, CR_ERR_STATE = -3, CR_ERR_NOMEM = -4 };
 enum { CR_BF16 = 0, CR_F32 = 1, CR_I64 = 2, CR_I32 = 3, CR_U8 = 4 /* library-internal: e4m3 weight copies */ };
@@ -167,22 +167,55 @@ int cr_llm_decode(cr_ctx* ctx, cr_kv* kv, const int32_t* seqs, int n, const int6
 /* A decoder-only language model whose layers are listed at run time: sizes, constants and the order of mechanisms come from these two structs (filled from the checkpoint's
  * config.json by callireader_amd/config.py: DecoderSpec), the weights through cr_load_weight under the checkpoint's names, the derived layout at cr_finalize.
  * The cache (cr_kv_*), the greedy pick, repetition penalty and cr_llm_decode are the ones above. */
-enum { CR_MIX_LATENT = 1 };                  /* latent attention: c = rms(W_dkv h), q = W_uq rms(W_dq h), k = W_uk c, v = W_uv c, sigmoid output gate; c is what is cached */
-enum { CR_FF_NONE = 0, CR_FF_MOE = 1 };      /* clamped gated experts behind a softmax router with a choice correction and expert groups */
+enum {
+    CR_MIX_LATENT = 1,                       /* latent attention: c = rms(W_dkv h), q = W_uq rms(W_dq h), k = W_uk c, v = W_uv c, sigmoid output gate; c is what is cached */
+    CR_MIX_HEADS = 2,                        /* softmax attention over grouped heads (cr_lm_heads) */
+    CR_MIX_RETENTION = 4,                    /* linear attention with a fixed decay per head (cr_lm_retention); HEADS | RETENTION: both on the same input, outputs added */
+};
+enum { CR_FF_NONE = 0, CR_FF_MOE = 1,        /* clamped gated experts behind a softmax router with a choice correction and expert groups */
+       CR_FF_DENSE = 2 };                    /* W_down act(W_up h) of width expert_ff */
+enum { CR_ACT_RELU2 = 1 };                   /* max(z, 0)^2 */
 enum { CR_POS_NONE = 0, CR_POS_SINUSOID = 1 };
+/* Rotations turn entries i and i + rot_dims / 2 of a head by position * rot_base^(-2 i / rot_dims); entries from rot_dims on stay (0: no rotation). */
+typedef struct cr_lm_heads {
+    char name[16];                           /* tensors l<i>.mix.<name>q, k, v, o, q.norm, k.norm */
+    int32_t heads, kv_heads, dim, vdim;      /* query head h reads key / value head h / (heads / kv_heads) */
+    int32_t chunk;                           /* > 0: a position sees keys of its own chunk of this many positions (counted from the sequence's first); 0: every earlier key */
+    int32_t qk_norm;                         /* RMS norm over each query and key head before the rotation */
+    int32_t rot_dims, reserved;
+    double rot_base;
+    float scale, softcap;                    /* score = (q . k) * scale, then softcap * tanh(score / softcap) when softcap > 0 */
+    float out_scale, reserved_f;             /* the mixer's output times this */
+} cr_lm_heads;
+typedef struct cr_lm_retention {
+    char name[16];                           /* tensors l<i>.mix.<name>q, k, v, g, o */
+    int32_t heads, dim, vdim, rot_dims;      /* S <- decay S + k v^T, o = S^T q; o over its root mean square per head, times silu(g) */
+    double rot_base;
+    float k_scale, out_scale;                /* keys times k_scale after the rotation */
+    const double* decay;                     /* [heads], read during cr_lm_configure */
+} cr_lm_retention;
 typedef struct cr_lm_layer {
-    int32_t mixer, heads, dim, vdim, q_rank, kv_rank;
+    int32_t mixer;                           /* CR_MIX_* */
+    int32_t heads, dim, vdim, q_rank, kv_rank;   /* CR_MIX_LATENT */
     float scale;                             /* score = (q . k) * scale */
     int32_t ff, experts, top, expert_ff, groups, keep;
     float limit;                             /* gate <= limit, |up| <= limit */
-    int32_t reserved[8];
+    int32_t act;                             /* CR_FF_DENSE: CR_ACT_* */
+    int32_t reserved[7];
+    cr_lm_heads attn;                        /* CR_MIX_HEADS */
+    cr_lm_retention ret;                     /* CR_MIX_RETENTION */
 } cr_lm_layer;
 typedef struct cr_lm_desc {
     int32_t layers, width, vocab, dtype;     /* dtype: CR_BF16, or CR_F32 = every product in true 32-bit */
-    int32_t loop_start, loop_stop, loop_times;   /* layers [start, stop) run `times` times in a row, each pass with a cache of its own; times = 0: no loop */
+    int32_t loop_start, loop_stop, loop_times;   /* layers [start, stop) run `times` times in a row, each pass with a cache or state of its own; times = 0: no loop */
     int32_t pos;                             /* CR_POS_SINUSOID: added to the embedding */
     float pos_base, eps, softcap;            /* softcap: logits <- softcap * tanh(logits / softcap); 0 = off */
-    int32_t reserved[8];
+    int32_t norm_plain;                      /* the model's norms multiply by their weight; 0: by one plus their weight */
+    int32_t no_post_norm;                    /* sublayer outputs join the residual as they are; 0: through a norm of their own (norm1b, norm2b) */
+    int32_t tied_head;                       /* logits from the embedding table (no tensor 'head') */
+    int32_t loop_in;                         /* x <- W [x; embedding] ahead of every pass of the looped span (tensor 'loop.in') */
+    int32_t side_dim;                        /* > 0: every layer ends with x += rms(W_proj (gelu_tanh(W_gate x) * e)) * w, e = its side_dim entries of the token's row of 'side.embed' */
+    int32_t reserved[7];
 } cr_lm_desc;
 /* After cr_create, before the weights: makes the context's language model the described one. */
 int cr_lm_configure(cr_ctx* ctx, const cr_lm_desc* desc, const cr_lm_layer* layers);
