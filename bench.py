@@ -89,8 +89,8 @@ def main():
     ap.add_argument('--fp8-extras', action='store_true', help='also time the batched decode on e4m3 weight copies alone (fp8_decode) and compare its first picks with the bf16 decode')
     ap.add_argument('--no-api', action='store_true', help='N = 1: skip the api_level block (the same batch from JPEG files through chat_ocr_stream / folder_rec to strings)')
     ap.add_argument('--api-batches', type=int, default=6, help='batches of --pages pages the api_level block streams')
-    ap.add_argument('--workload', choices=('pages', 'linasun'), default='pages', help='linasun: prefill and decode of the described decoder beside InternLM2 layers (benchlib/decoder.py), N = 1')
-    ap.add_argument('--sizes', default=None, help='--workload linasun: comma-separated subset of its sizes')
+    ap.add_argument('--workload', choices=('pages', 'linasun', 'lugasun'), default='pages', help='linasun, lugasun: prefill and decode of that described decoder beside InternLM2 layers (benchlib/decoder.py), N = 1')
+    ap.add_argument('--sizes', default=None, help='--workload linasun | lugasun: comma-separated subset of its sizes')
     ap.add_argument('--no-pipeline', action='store_true', help='one batch at a time (the decode of a batch does not run beside the visual stage of the next)')
     args = ap.parse_args()
     plan.NEW_TOKENS = NEW_TOKENS = args.new_tokens
@@ -113,11 +113,11 @@ def main():
     local_rank = local_rank % n_dev
     torch.cuda.set_device(local_rank)
     dev = torch.device('cuda', local_rank)
-    if args.workload == 'linasun':
+    if args.workload != 'pages':
         from benchlib import decoder
         if world != 1:
-            raise SystemExit('--workload linasun runs on one GPU')
-        return decoder.main(dev, args.sizes.split(',') if args.sizes else None)
+            raise SystemExit(f'--workload {args.workload} runs on one GPU')
+        return decoder.main(args.workload, dev, args.sizes.split(',') if args.sizes else None)
     if world > 1:
         os.environ.setdefault('HSA_ENABLE_IPC_MODE_LEGACY', '0')
         if backend == 'nccl':

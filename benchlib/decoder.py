@@ -1,5 +1,5 @@
-"""`bench.py --workload linasun`: prefill and decode throughput of the described decoder (Linasun) at a few sizes that resemble a real model's layers, random weights, beside the
-engine's InternLM2 layers at equal width and equal active feed-forward width.  One process, one GPU; HIP events on the current stream; prints one JSON line."""
+"""`bench.py --workload linasun | lugasun`: prefill and decode throughput of a described decoder at a few sizes that resemble a real model's layers, random weights, beside the
+engine's InternLM2 layers at equal width and equal (active) feed-forward weights.  One process, one GPU; HIP events on the current stream; prints one JSON line."""
 import json
 import math
 
@@ -18,11 +18,28 @@ def _cfg(width, heads, dim, q_rank, kv_rank, experts, top, ff, groups, layers, v
                 **({'loop': dict(start=loop[0], stop=loop[1], times=loop[2])} if loop else {}))
 
 
-SIZES = {
+LINASUN = {
     'w4096_e64': _cfg(4096, 32, 128, 1536, 512, 64, 8, 1792, (8, 4), 4, 92553),          # active feed-forward width 8 x 1792 = InternLM2.5-7B's 14336
     'w2048_e32': _cfg(2048, 16, 128, 768, 512, 32, 4, 1024, (4, 2), 8, 32000),
     'w1024_looped': _cfg(1024, 8, 128, 384, 256, 16, 2, 1024, (4, 2), 6, 32000, loop=(1, 5, 3)),
 }
+
+
+def _lugasun(width, heads, kv_heads, dim, chunk, ret_heads, ret_dim, ret_vdim, ff, side, layers, vocab, loop=None):
+    left = dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=dim, mask=dict(size=chunk), scale=dim ** -0.5, softcap=50.0, rot=dict(base=1e6, dims=dim))
+    right = dict(heads=ret_heads, dim=ret_dim, vdim=ret_vdim, decay=[1.0 - 2.0 ** (-5 - 6 * i / ret_heads) for i in range(ret_heads)], rot=dict(base=1e4, dims=ret_dim))
+    layer = dict(type='parallel', mixer=dict(left=left, right=right, left_scale=0.7, right_scale=0.7), mlp=dict(kind='dense', ff=ff))
+    return dict(architecture='Lugasun', width=width, vocab=vocab, norm=dict(eps=1e-6), layers=[layer] * layers, token_side=dict(dim=side),
+                **({'loop': dict(start=loop[0], stop=loop[1], times=loop[2])} if loop else {}))
+
+
+LUGASUN = {
+    # attention heads, cached keys and feed-forward weights (2 x 21504 rows against 3 x 14336) are InternLM2.5-7B's; retention and the token side come on top
+    'w4096_c8192': _lugasun(4096, 32, 8, 128, 8192, 32, 128, 128, 21504, 256, 4, 92553),
+    'w2048_c1024': _lugasun(2048, 16, 4, 128, 1024, 8, 128, 256, 8192, 128, 8, 32000),
+    'w1024_looped': _lugasun(1024, 8, 2, 128, 512, 8, 64, 64, 4096, 64, 6, 32000, loop=(1, 5, 3)),
+}
+SIZES = {'linasun': LINASUN, 'lugasun': LUGASUN}
 
 
 def random_weights(spec, device, seed=0):
@@ -32,39 +49,82 @@ def random_weights(spec, device, seed=0):
         leaf = name.rsplit('.', 1)[-1]
         r = torch.randn(*shape, device=device, generator=g)
         if len(shape) == 1:
-            r = 1.0 + 0.1 * r if leaf == 'norm' and name != 'final.norm' else (1e-3 if leaf == 'correction' else 0.1) * r      # (small corrections: balanced experts)
+            r = 1.0 + 0.1 * r if spec.norm_plain or (leaf == 'norm' and name != 'final.norm') else (1e-3 if leaf == 'correction' else 0.1) * r      # (small corrections: balanced experts)
         elif name != 'embed':
             r = r / math.sqrt(shape[1])
         yield name, r.to(torch.bfloat16)
 
 
-def linasun(cfg, max_tokens, rows, device=0, dtype=torch.bfloat16):
-    from callireader_amd.config import DecoderSpec
-    from callireader_amd.modeling_decoder import LinasunForCausalLM
-    spec = DecoderSpec.from_linasun(cfg)
-    return LinasunForCausalLM.from_state_dict(random_weights(spec, torch.device('cuda', device)), spec, device=device, dtype=dtype, max_tokens=max_tokens, max_seqs=rows)
+def build(cfg, max_tokens, rows, device=0, dtype=torch.bfloat16):
+    from callireader_amd import modeling_decoder, registry
+    cls = getattr(modeling_decoder, registry.MODELS[cfg['architecture']][1])
+    spec = cls.read_config(cfg)
+    return cls.from_state_dict(random_weights(spec, torch.device('cuda', device)), spec, device=device, dtype=dtype, max_tokens=max_tokens, max_seqs=rows)
+
+
+def _visible(n, chunk):
+    """Keys that positions 0 .. n - 1 see, in all."""
+    full, rest = divmod(n, chunk) if chunk else (0, n)
+    return full * chunk * (chunk + 1) / 2 + rest * (rest + 1) / 2
+
+
+def _mixers(m):
+    from callireader_amd.config import ParallelMixer
+    return [m.left, m.right] if isinstance(m, ParallelMixer) else [m]
+
+
+def _ff_weights(spec, f, rows=None):
+    """Feed-forward weights a token multiplies (rows=None), or that a batch of `rows` tokens reads (every expert some row is expected to choose, uniform choices)."""
+    from callireader_amd.config import DenseFF
+    if f is None:
+        return 0
+    if isinstance(f, DenseFF):
+        return 2 * spec.width * f.ff
+    return spec.width * f.experts + (f.top if rows is None else f.experts * (1 - (1 - f.top / f.experts) ** rows)) * 3 * spec.width * f.ff
+
+
+def _mixer_weights(spec, m):
+    from callireader_amd.config import HeadsMixer, RetentionMixer
+    if isinstance(m, HeadsMixer):
+        return spec.width * (m.heads * (m.dim + m.vdim) + m.kv_heads * (m.dim + m.vdim))
+    if isinstance(m, RetentionMixer):
+        return spec.width * m.heads * (2 * m.dim + 3 * m.vdim)
+    return spec.width * (m.q_rank + m.kv_rank + 2 * m.heads * m.vdim) + m.q_rank * m.heads * m.dim + m.kv_rank * m.heads * (m.dim + m.vdim)
+
+
+def _loop_weights(spec):
+    return (spec.loop[2] if spec.loop_in and spec.loop else 0) * 2 * spec.width * spec.width
 
 
 def prefill_flops(spec, tokens, seqs):
-    """2 x multiply-adds of the equations as written (keys and values formed once per token), causal half of the attention, logits of the last rows."""
-    f = 0.0
+    """2 x multiply-adds of the equations as written (keys and values formed once per token, retention as its recurrence), visible keys of the attention, logits of the last rows."""
+    from callireader_amd.config import HeadsMixer, RetentionMixer
+    f = 2.0 * tokens * _loop_weights(spec)
     for i in spec.passes:
-        m, e = spec.layers[i].mixer, spec.layers[i].ff
-        f += 2.0 * tokens * (spec.width * (m.q_rank + m.kv_rank + m.heads * m.vdim) + m.q_rank * m.heads * m.dim + m.kv_rank * m.heads * (m.dim + m.vdim) + m.heads * m.vdim * spec.width)
-        f += 2.0 * seqs * (tokens / seqs) * (tokens / seqs + 1) / 2 * m.heads * (m.dim + m.vdim)
-        if e:
-            f += 2.0 * tokens * (spec.width * e.experts + e.top * 3 * spec.width * e.ff)
+        for m in _mixers(spec.layers[i].mixer):
+            f += 2.0 * tokens * _mixer_weights(spec, m)
+            if isinstance(m, RetentionMixer):
+                f += 2.0 * tokens * m.heads * 2 * m.dim * m.vdim
+            else:
+                f += 2.0 * seqs * _visible(tokens // seqs, m.chunk if isinstance(m, HeadsMixer) else 0) * m.heads * (m.dim + m.vdim)
+        f += 2.0 * tokens * (_ff_weights(spec, spec.layers[i].ff) + 2 * spec.width * spec.side_dim)
     return f + 2.0 * seqs * spec.width * spec.vocab
 
 
 def decode_bytes(spec, rows, ctx):
-    """Weights and cache a decode step has to read once: every expert some row is expected to choose (uniform choices), the rows' latents."""
-    b = 2.0 * spec.width * spec.vocab
+    """Weights and cache a decode step has to read once, and the states it reads and writes."""
+    from callireader_amd.config import HeadsMixer, RetentionMixer
+    b = 2.0 * spec.width * spec.vocab + 2.0 * _loop_weights(spec)
     for i in spec.passes:
-        m, e = spec.layers[i].mixer, spec.layers[i].ff
-        b += 2.0 * (spec.width * (m.q_rank + m.kv_rank + 2 * m.heads * m.vdim) + m.q_rank * m.heads * m.dim + m.kv_rank * m.heads * (m.dim + m.vdim)) + 2.0 * rows * ctx * m.kv_rank
-        if e:
-            b += 2.0 * (spec.width * e.experts + e.experts * (1 - (1 - e.top / e.experts) ** rows) * 3 * spec.width * e.ff)
+        for m in _mixers(spec.layers[i].mixer):
+            b += 2.0 * _mixer_weights(spec, m)
+            if isinstance(m, RetentionMixer):
+                b += 8.0 * rows * m.heads * m.dim * m.vdim
+            elif isinstance(m, HeadsMixer):
+                b += 2.0 * rows * (ctx % m.chunk + 1 if m.chunk else ctx) * m.kv_heads * (m.dim + m.vdim)
+            else:
+                b += 2.0 * rows * ctx * m.kv_rank
+        b += 2.0 * (_ff_weights(spec, spec.layers[i].ff, rows) + 2 * spec.width * spec.side_dim)
     return b
 
 
@@ -99,9 +159,8 @@ def measure(kv, prefill, decode, flops, bytes_of, steps=20):
     return out
 
 
-def run_linasun(name, dev):
-    cfg = SIZES[name]
-    m = linasun(cfg, CTX + 3 * 25, max(ROWS), dev.index)
+def run_size(workload, name, dev):
+    m = build(SIZES[workload][name], CTX + 3 * 25, max(ROWS), dev.index)
     e, spec = m.engine, m.spec
     kv = e.kv_alloc(max(ROWS), CTX + 3 * 25)
     g = torch.Generator().manual_seed(1)
@@ -137,22 +196,29 @@ def run_internlm2(dev, layers=4):
     return out
 
 
-def run(dev, only=None):
+def _describe(workload, c):
+    layer = c['layers'][0]
+    d = dict(width=c['width'], layers=len(c['layers']), loop=c.get('loop'), vocab=c['vocab'])
+    if workload == 'lugasun':
+        left, right = layer['mixer']['left'], {k: v for k, v in layer['mixer']['right'].items() if k not in ('decay', 'rot')}
+        return dict(d, attention={k: v for k, v in left.items() if k not in ('rot', 'mask')}, chunk=left['mask']['size'], retention=right, ff=layer['mlp']['ff'], token_side=c['token_side']['dim'])
+    return dict(d, **layer['mixer'], experts=layer['mlp']['router']['experts'], top=layer['mlp']['router']['top'], expert_ff=layer['mlp']['expert']['ff'])
+
+
+def run(workload, dev, only=None):
     res = {}
     with torch.inference_mode():
         if not only or 'internlm2' in only:
             res['internlm2_4_layers'] = run_internlm2(dev)
-        for name in SIZES:
+        for name in SIZES[workload]:
             if not only or name in only:
-                res[name] = run_linasun(name, dev)
+                res[name] = run_size(workload, name, dev)
                 torch.cuda.empty_cache()
-    ref = res.get('w4096_e64') or next(v for k, v in res.items())
-    return {'metric': 'Linasun layers: decode tokens/s (64 rows, 4 layers of width 4096)', 'value': ref['decode']['64']['tokens_per_s'], 'unit': 'tokens/s', 'n_gpus': 1, 'higher_is_better': True,
-            'vs_baseline': None, 'dtype': 'bf16', 'data': 'synthetic', 'sizes': res,
-            'config': {k: dict(width=c['width'], layers=len(c['layers']), loop=c.get('loop'), **c['layers'][0]['mixer'], experts=c['layers'][0]['mlp']['router']['experts'],
-                               top=c['layers'][0]['mlp']['router']['top'], expert_ff=c['layers'][0]['mlp']['expert']['ff'], vocab=c['vocab']) for k, c in SIZES.items()},
+    ref = res.get(next(iter(SIZES[workload]))) or next(v for k, v in res.items())
+    return {'metric': f'{workload.capitalize()} layers: decode tokens/s (64 rows, 4 layers of width 4096)', 'value': ref['decode']['64']['tokens_per_s'], 'unit': 'tokens/s', 'n_gpus': 1,
+            'higher_is_better': True, 'vs_baseline': None, 'dtype': 'bf16', 'data': 'synthetic', 'sizes': res, 'config': {k: _describe(workload, c) for k, c in SIZES[workload].items()},
             'how': 'HIP events around whole engine calls after a warm-up call; flops and bytes are algorithmic (this file), peaks as everywhere in bench.py'}
 
 
-def main(dev, only=None):
-    print(json.dumps(run(dev, only)), flush=True)
+def main(workload, dev, only=None):
+    print(json.dumps(run(workload, dev, only)), flush=True)
