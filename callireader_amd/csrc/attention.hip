@@ -20,6 +20,7 @@
 #include <type_traits>
 
 #include "attention.hpp"
+#include "attention_merge.hpp"
 
 namespace {
 
@@ -433,41 +434,8 @@ int launch_t(const AttnParams& p, hipStream_t stream) {
     return p.s_div != 1.0f ? launch_d<D, CAUSAL, true>(p, stream) : launch_d<D, CAUSAL, false>(p, stream);
 }
 
-// out[b][q][h][:] = sum_s exp(m_s - M) O_s / sum_s exp(m_s - M) l_s   (splits in index order: reproducible)
-// A wave's lane s fetches split s's (m, l) -- one round trip for up to 64 splits, maximum and weights by shuffles -- and the O rows are
-// loaded eight at a time with independent loads (a plain loop over the run-time split count waited for every load in turn: 13
-// dependent round trips per launch at 3 300 cached tokens, 11.5 us x 32 layers per decode step).
 template <int D>
-__global__ __launch_bounds__(D) void attn_combine_kernel(const AttnParams p) {
-    const int q = blockIdx.x, head = blockIdx.y, batch = blockIdx.z, d = threadIdx.x, lane = d & 63;
-    const int64_t base = ((int64_t)batch * p.H + head) * p.nsplit;
-    float M = -INFINITY;
-    for (int s0 = 0; s0 < p.nsplit; s0 += 64) {
-        const int s = s0 + lane;
-        M = fmaxf(M, wave_max(s < p.nsplit ? p.part_ml[((base + s) * p.Sq + q) * 2] : -INFINITY));
-    }
-    float L = 0.f, acc = 0.f;
-    for (int s0 = 0; s0 < p.nsplit; s0 += 64) {
-        const int s = s0 + lane;
-        const bool in = s < p.nsplit;
-        const int64_t row = (base + (in ? s : 0)) * p.Sq + q;
-        const float w = in ? __expf(p.part_ml[row * 2] - M) : 0.f;
-        const float wl = in ? w * p.part_ml[row * 2 + 1] : 0.f;
-        const int n = min(64, p.nsplit - s0);
-        for (int j0 = 0; j0 < n; j0 += 8) {
-            float o[8];
-#pragma unroll
-            for (int j = 0; j < 8; j++) o[j] = j0 + j < n ? p.part_o[((base + s0 + j0 + j) * p.Sq + q) * D + d] : 0.f;
-#pragma unroll
-            for (int j = 0; j < 8; j++) {                    // index order; lanes past the count carry weight 0
-                L += __shfl(wl, j0 + j, 64);
-                acc += __shfl(w, j0 + j, 64) * o[j];
-            }
-        }
-    }
-    if (p.wide && d >= p.vdim) return;
-    p.O[(int64_t)batch * p.o_bs + (int64_t)q * p.o_rs + (int64_t)head * p.o_hs + d] = f2bf(p.wide && p.out_mul != 0.f ? p.out_mul * acc / L : acc / L);
-}
+__global__ __launch_bounds__(D) void attn_combine_kernel(const AttnParams p) { attn_merge_splits(p, D, blockIdx.z, blockIdx.y, blockIdx.x, threadIdx.x); }
 
 template <int D, bool DIV>
 int launch_split_d(const AttnParams& p, hipStream_t stream) {
@@ -482,7 +450,7 @@ int launch_split_d(const AttnParams& p, hipStream_t stream) {
 template <int D>
 int launch_split_wide(const AttnParams& p, hipStream_t stream) {
     const int rc = p.softcap > 0.f ? launch_wide<D, false, true, 2>(p, stream) : launch_wide<D, false, true, 1>(p, stream);
-    if (rc != CR_OK) return rc;
+    if (rc != CR_OK || p.no_merge) return rc;
     hipLaunchKernelGGL((attn_combine_kernel<D>), dim3(p.Sq, p.H, p.B), dim3(D), 0, stream, p);
     return hipGetLastError() == hipSuccess ? CR_OK : CR_ERR_HIP;
 }

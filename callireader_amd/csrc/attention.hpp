@@ -40,6 +40,7 @@ struct AttnParams {
     int wide;
     float s_mul;              // > 0
     float softcap, out_mul;
+    bool no_merge;            // decode: leave the partials, the caller merges them (attention_merge.hpp)
     int sk_mod;               // decode: > 0: a row sees the last sk_arr[slot] % sk_mod + sk_add keys, which start at its slot's first row
     int vdim;
     const bf16* gate; int64_t g_rs;

@@ -171,6 +171,7 @@ enum GemmEpi {
     EPI_X_GLU = 10,   // grouped experts (gemm256 only): rows gathered through `perm`, W rows interleaved [8 gate | 8 up], clamped gated unit (GemmParams::limit)
     EPI_X_ROWS = 11,  // grouped experts (gemm256 only): plain rows, scattered through `perm`
     EPI_RELU2 = 12,   // bf16(max(acc, 0)^2), no bias
+    EPI_SIDE = 13,    // 128-row kernel only: bf16(gelu_tanh(acc) * res[perm[m]][n]): a gate times a row looked up by the token
     EPI_ARGMAX = 8,   // cosine VQ: C[m][b] = {col, bits(max)} of bf16(acc) over the 64 columns of block b (first max wins); nothing else stored
 };
 

@@ -186,6 +186,7 @@ int launch_gemm(int epi, const GemmParams& p, hipStream_t stream) {
         case EPI_STORE: return launch_t<EPI_STORE>(p, stream);
         case EPI_GELU: return launch_t<EPI_GELU>(p, stream);
         case EPI_RELU2: return launch_t<EPI_RELU2>(p, stream);
+        case EPI_SIDE: return (p.res && p.perm && (p.ldr & 7) == 0 && ((uintptr_t)p.res & 15) == 0 && p.N % 8 == 0) ? launch_t<EPI_SIDE>(p, stream) : CR_ERR_ARG;
         case EPI_LS_RES: return (p.scale && p.res) ? launch_t<EPI_LS_RES>(p, stream) : CR_ERR_ARG;
         case EPI_RES: return p.res ? launch_t<EPI_RES>(p, stream) : CR_ERR_ARG;
         case EPI_SWIGLU: return (p.N % 16 == 0) ? launch_t<EPI_SWIGLU>(p, stream) : CR_ERR_ARG;

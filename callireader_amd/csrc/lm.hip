@@ -21,6 +21,8 @@
 #include "kv.hpp"
 #include "lm.hpp"
 
+bool gemm_stream_supported(int epi, const GemmParams& p, int splits);      // gemm_stream.hip
+
 namespace {
 
 // Re-laid-out, padded, converted copies of checkpoint tensors (load time): src row r goes to row d = r, or to row 16 (r / 8) + r % 8 + row_off when interleaved in eights;
@@ -269,7 +271,7 @@ Buffers carve(const Lm& lm, Arena& ar, const Step& sp) {
     const int M = sp.M, Wp = lm.Wp;
     const bool decode = sp.decode, sliced = decode && !lm.f32 && M <= 64;
     size_t Na = 0, Qp = 0, Rp = 0, Gp = 0, qn = 0, kvn = 0, hr = 0, Ep = 0, top = 0, act = 0, tiles = 0, part = 0, sl = 0, kvh = 0, r32 = 0, r16 = 0, raw = 0, snap = 0;
-    auto slices = [&](int N, int K) { if (sliced) sl = std::max(sl, (size_t)M * gemm_partial_splits(N, K) * N); };
+    auto slices = [&](int N, int K) { if (sliced) sl = std::max(sl, (size_t)M * std::max(1, gemm_partial_splits(N, K)) * N); };
     for (const LmLayer& L : lm.layers) {
         Na = std::max<size_t>(Na, L.Na); Gp = std::max<size_t>(Gp, L.Gp);
         slices(L.Na, Wp); slices(Wp, L.Gp);
@@ -318,12 +320,20 @@ size_t carve_bytes(const Lm& lm, const Step& sp) {
     return ar.off + 512;
 }
 
-// decode of <= 64 rows: fp32 K-slices of A . W^T (gemm_skinny.hip) for a consumer that adds them; 0 when the shape has no such form
-int slices_of(const Lm& lm, int M, int N, int K, bool decode) { return !lm.f32 && decode && M <= 64 ? gemm_partial_splits(N, K) : 0; }
-int sliced(cr_ctx* c, const void* A, int64_t lda, const void* W, const bf16* dl, float* C, int M, int N, int K, hipStream_t st) {
+// decode of <= 64 rows: fp32 K-slices of A . W^T (gemm_skinny.hip) for a consumer that adds them; 0 when the shape has no such form.  Wide products of more than a few rows are one
+// slice through the kernel that splits N over its waves (gemm_stream.hip).
+GemmParams slice_params(const void* A, int64_t lda, const void* W, const bf16* dl, float* C, int M, int N, int K) {
     GemmParams p{};
     p.A = (const bf16*)A; p.lda = lda; p.W = dl ? dl : (const bf16*)W; p.ldw = K; p.wsw = dl ? 1 : 0; p.C = C; p.ldc = N; p.M = M; p.N = N; p.K = K;
-    return ctx_gemm(c, EPI_PARTIAL, p, st);
+    return p;
+}
+bool one_slice(int M, int N, int K) { return gemm_stream_supported(EPI_F32, slice_params(nullptr, K, nullptr, nullptr, nullptr, M, N, K), 1); }
+int slices_of(const Lm& lm, int M, int N, int K, bool decode) { return lm.f32 || !decode || M > 64 ? 0 : one_slice(M, N, K) ? 1 : gemm_partial_splits(N, K); }
+int sliced(cr_ctx* c, const void* A, int64_t lda, const void* W, const bf16* dl, float* C, int M, int N, int K, hipStream_t st) {
+    GemmParams p = slice_params(A, lda, W, dl, C, M, N, K);
+    if (!one_slice(M, N, K)) return ctx_gemm(c, EPI_PARTIAL, p, st);
+    p.raw32 = 1;
+    return ctx_gemm(c, EPI_F32, p, st);
 }
 
 // C[M, N] = A . W^T in the model's element type: the engine's dense kernels for bf16, the fp32 tile kernel otherwise
@@ -425,10 +435,11 @@ int heads_mixer(cr_ctx* c, cr_kv* kv, const Step& sp, Buffers& b, const LmLayer&
     in.ring = ring; in.chunk = chunk; in.row_key = kp ? kp->row_key : nullptr; in.row_slot = kp ? kp->row_slot : nullptr; in.ao = b.ao;
     if (matrix) { in.rq2 = b.rq2; in.rk2 = b.rk2; } else { in.rq = b.rq; in.rk = b.rk; }
     CR_TRY(launch_lm_heads(lm.f32, lm, L, M, in, st));
+    AttnParams ap{};
+    bool merge = false;
     if (L.heads()) {
         const int64_t qld = (int64_t)a.heads * L.Ap, ldk = (int64_t)2 * a.kv_heads * L.Ap;
         if (flash_heads(lm, L)) {
-            AttnParams ap{};
             ap.Q = (const bf16*)b.q; ap.O = (bf16*)b.ao; ap.q_prescale = 1.f; ap.s_div = 1.f; ap.wide = 1; ap.s_mul = a.scale; ap.softcap = a.softcap; ap.out_mul = a.out_scale; ap.vdim = a.vdim;
             if (sp.decode) {
                 const int rows = heads_per_split(a), nsplit = sp.hsplit[L.chunk_ix];
@@ -436,6 +447,7 @@ int heads_mixer(cr_ctx* c, cr_kv* kv, const Step& sp, Buffers& b, const LmLayer&
                 ap.q_bs = qld; ap.q_rs = L.Ap; ap.q_hs = (int64_t)rows * L.Ap; ap.k_rs = ap.v_rs = L.Ap; ap.k_hs = ap.v_hs = (int64_t)ring * L.Ap; ap.k_bs = ap.v_bs = a.kv_heads * ap.k_hs;
                 ap.o_bs = L.Gp; ap.o_rs = a.vdim; ap.o_hs = (int64_t)rows * a.vdim; ap.seq_map = sp.ix.seqs; ap.sk_arr = sp.ix.lens; ap.sk_add = 1; ap.sk_mod = chunk;
                 ap.nsplit = nsplit; ap.part_o = b.part; ap.part_ml = b.part + (size_t)M * a.heads * nsplit * L.Ap;
+                ap.no_merge = merge = L.retention();          // retention's launch takes the merge along
                 if (launch_flash_attn_split(ap, L.Ap, st) != CR_OK) return cr_fail(CR_ERR_HIP, "attention over heads (decode): launch failed");
             } else {
                 ap.K = (const bf16*)b.kv; ap.V = (const bf16*)b.kv + (size_t)a.kv_heads * L.Ap;
@@ -461,7 +473,7 @@ int heads_mixer(cr_ctx* c, cr_kv* kv, const Step& sp, Buffers& b, const LmLayer&
     rp.ao = (char*)b.ao + (size_t)L.off_r * es; rp.ldo = L.Gp; rp.state = (float*)(kv->lat + kv->state_off[r]); rp.raw = b.raw; rp.snap = b.snap; rp.pw = L.pw;
     rp.M = M; rp.H = rt.heads; rp.Kp = L.Kp; rp.Vp = L.Vp; rp.vdim = rt.vdim; rp.eps = lm.d.eps; rp.out_scale = rt.out_scale; rp.ix = sp.ix;
     rp.seg = sp.d_rseg; rp.snap0 = sp.d_snap0; rp.n_segs = (int)sp.segs.size(); rp.longest = sp.longest;
-    return sp.decode ? launch_ret_decode(lm.f32, rp, st) : matrix ? launch_ret_matrix(rp, st) : launch_ret_recurrent(lm.f32, rp, st);
+    return sp.decode ? launch_ret_decode(lm.f32, rp, merge ? &ap : nullptr, L.Ap, st) : matrix ? launch_ret_matrix(rp, st) : launch_ret_recurrent(lm.f32, rp, st);
 }
 
 // h -> ye, wt: the rows of every chosen expert and their weights
@@ -558,6 +570,11 @@ int run_passes(cr_ctx* c, cr_kv* kv, const Step& sp, Buffers& b, hipStream_t st)
             if (n) {
                 CR_TRY(sliced(c, b.h, Wp, L.sgate, L.sgate_dl, b.sl, M, lm.Sp, Wp, st));
                 CR_TRY(launch_lm_side_act(lm, M, b.sl, n, side, lds, b.tok, b.z2, st));
+            } else if (!lm.f32) {
+                GemmParams g{};
+                g.A = (const bf16*)b.h; g.lda = Wp; g.W = (const bf16*)L.sgate; g.ldw = Wp; g.C = b.z2; g.ldc = lm.Sp; g.M = M; g.N = lm.Sp; g.K = Wp; g.kernel = 128;
+                g.res = (const bf16*)side; g.ldr = lds; g.perm = b.tok;
+                CR_TRY(ctx_gemm(c, EPI_SIDE, g, st));
             } else {
                 LmGemmParams g{};
                 g.A = b.h; g.lda = Wp; g.W = L.sgate; g.ldw = Wp; g.C = b.z2; g.ldc = lm.Sp; g.M = M; g.N = lm.Sp; g.K = Wp; g.gate = side; g.ldg = lds; g.tok = b.tok;

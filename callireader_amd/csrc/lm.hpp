@@ -7,6 +7,7 @@
 #include <string>
 #include <vector>
 
+#include "attention.hpp"
 #include "common.hpp"
 #include "ctx.hpp"
 
@@ -213,7 +214,8 @@ struct RetParams {
 };
 bool ret_matrix_supported(int Kp, int Vp);
 inline int ret_snapshots(int rows) { return (rows + RET_CHUNK - 1) / RET_CHUNK; }
-int launch_ret_decode(bool f32, const RetParams& p, hipStream_t st);
+// merge: decode splits that the attention beside it left (AttnParams::no_merge), of heads of merge_dim columns
+int launch_ret_decode(bool f32, const RetParams& p, const AttnParams* merge, int merge_dim, hipStream_t st);
 int launch_ret_recurrent(bool f32, const RetParams& p, hipStream_t st);
 int launch_ret_matrix(const RetParams& p, hipStream_t st);
 // decode of <= 64 rows: z[m][n] = gelu_tanh(sum of K-slices) * side[tok[m]][n]

@@ -276,7 +276,13 @@ __global__ __launch_bounds__(256) void lm_side_act_kernel(const float* __restric
     if (i >= M * Sp) return;
     const int m = i / Sp, n = i - m * Sp;
     f32x4 s = {0.f, 0.f, 0.f, 0.f};
-    for (int k = 0; k < slices; k++) s += *(const f32x4*)(part + ((int64_t)k * M + m) * Sp + n);
+    for (int k = 0; k < slices; k += 8) {
+        f32x4 v[8];
+#pragma unroll
+        for (int q = 0; q < 8; q++) v[q] = k + q < slices ? *(const f32x4*)(part + ((int64_t)(k + q) * M + m) * Sp + n) : f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int q = 0; q < 8; q++) s += v[q];
+    }
     const f32x4 e = ld4(side + (int64_t)tok[m] * lds + n);
     st4(z + i, f32x4{gelu_tanh(s[0]) * e[0], gelu_tanh(s[1]) * e[1], gelu_tanh(s[2]) * e[2], gelu_tanh(s[3]) * e[3]});
 }

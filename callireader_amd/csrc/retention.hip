@@ -10,6 +10,7 @@
 // Powers of the decay come from a table in fp32 made from double (decay^0 .. decay^RET_CHUNK): no logarithm, so decays of 0 and 1 are ordinary.
 //
 // Prompts in fp32, and sizes past the matrix form: the recurrence token by token, state in registers, then a norm-and-gate kernel.
+#include "attention_merge.hpp"
 #include "lm.hpp"
 
 namespace {
@@ -36,11 +37,17 @@ __device__ __forceinline__ float silu32(float x) { return x / (1.0f + expf(-x));
 
 constexpr int dec_waves(int NR) { return NR > 16 ? 8 : 16; }
 
+// workgroups past the heads merge the attention's key splits of the same row (the mixer beside this one), a wave per 64 columns: two short launches in one
 template <typename T, int NR>
-__global__ __launch_bounds__(dec_waves(NR) * 64) void ret_decode_kernel(const RetParams p) {
+__global__ __launch_bounds__(dec_waves(NR) * 64) void ret_decode_kernel(const RetParams p, const AttnParams merge, int merge_dim) {
     __shared__ float so[LM_MAX_HEAD], red[LM_MAX_HEAD / 16];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, nw = blockDim.x >> 6;
     const int h = blockIdx.x, row = blockIdx.y;
+    if (h >= p.H) {
+        const int u = (h - p.H) * nw + wave, parts = merge_dim / 64, hq = u / parts;
+        if (hq < merge.H * merge.Sq) attn_merge_splits(merge, merge_dim, row, hq / merge.Sq, hq % merge.Sq, (u % parts) * 64 + lane);
+        return;
+    }
     const int seq = p.ix.seqs[row];
     const bool fresh = p.ix.lens[seq] == 0;                   // a state starts at zero, whatever the slot held before
     const int g = lane >> 2, c4 = (lane & 3) * 4, blocks = p.Vp >> 4;
@@ -154,7 +161,10 @@ __device__ __forceinline__ bf16x8 read_tr(const char* at, int row_bytes) {
     return bf16x8{lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]};
 }
 
-// S^T[64 dv][64 dk] of one (segment, head), 64 rows of the segment at a time: S^T <- decay^n S^T + V^T (decay^(n-1-j) k_j)
+// snapshot of a (chunk, head), two terms of [Vp / 32][Kp / 16] blocks of 1 KiB: S^T as ret_out_kernel's A operand (lane = value column % 32, + 32 for the second eight dk)
+__device__ __forceinline__ int64_t ret_snap_at(int dk, int dv, int Kp) { return ((int64_t)(dv >> 5) * (Kp >> 4) + (dk >> 4)) * 512 + ((dv & 31) + ((dk & 8) << 2)) * 8 + (dk & 7); }
+
+// S[64 dk][64 dv] of one (segment, head), 64 rows of the segment at a time: S <- decay^n S + (decay^(n-1-j) k_j)^T V.  Two tiles of loads are under way while one is multiplied.
 __global__ __launch_bounds__(256) void ret_state_kernel(const RetParams p) {
     __shared__ __attribute__((aligned(16))) char sm[2][3][8192];          // [buffer][v, k, k's remainder][64 rows][64 columns]
     const int tid = threadIdx.x, lane = tid & 63;
@@ -166,62 +176,63 @@ __global__ __launch_bounds__(256) void ret_state_kernel(const RetParams p) {
     const int64_t plane = (int64_t)p.M * p.H * p.Kp;
     const int l31 = lane & 31, hh = lane >> 5, wv = wave & 1, wk = wave >> 1;
     float* st = p.state + ((int64_t)seq * p.H + h) * p.Vp * p.Kp;
-    const int NR = p.Kp / 16, dk = kt * 64 + wk * 32 + l31, dv0 = vt * 64 + wv * 32 + 4 * hh;
+    const int NR = p.Kp / 16, dv = vt * 64 + wv * 32 + l31, dk0 = kt * 64 + wk * 32 + 4 * hh;      // lane: value column dv, element e: dk0 + (e & 3) + 8 (e >> 2)
     f32x16 acc;
 #pragma unroll
-    for (int e = 0; e < 16; e++) acc[e] = sg[2] == 0 ? 0.f : st[ret_state_at(dk, dv0 + (e & 3) + 8 * (e >> 2), NR)];
+    for (int e = 0; e < 16; e++) acc[e] = sg[2] == 0 ? 0.f : st[ret_state_at(dk0 + (e & 3) + 8 * (e >> 2), dv, NR)];
 
     // staging: a thread carries 16 columns of one row
     const int r = tid >> 2, c0 = (tid & 3) * 2;
     const bf16* vp = (const bf16*)p.v + (int64_t)row0 * p.lda + h * p.Vp + vt * 64 + c0 * 8;
     const bf16* kp = p.rk2 + ((int64_t)row0 * p.H + h) * p.Kp + kt * 64 + c0 * 8;
-    bf16x8 v[2], a[2], b[2];
-    auto load = [&](int t) {
+    struct Tile { bf16x8 v[2], a[2], b[2]; float w; };
+    const int nt = (S + 63) / 64;
+    auto load = [&](int t, Tile& x) {
         const int64_t q = min(t * 64 + r, S - 1);
+        const int n = min(64, S - t * 64);
+        x.w = r < n ? pw[n - 1 - r] : 0.f;
 #pragma unroll
         for (int i = 0; i < 2; i++) {
-            v[i] = *(const bf16x8*)(vp + q * p.lda + i * 8);
-            a[i] = *(const bf16x8*)(kp + q * p.H * p.Kp + i * 8);
-            b[i] = *(const bf16x8*)(kp + plane + q * p.H * p.Kp + i * 8);
+            x.v[i] = *(const bf16x8*)(vp + q * p.lda + i * 8);
+            x.a[i] = *(const bf16x8*)(kp + q * p.H * p.Kp + i * 8);
+            x.b[i] = *(const bf16x8*)(kp + plane + q * p.H * p.Kp + i * 8);
         }
     };
-    auto store = [&](int t, int buf) {
-        const int n = min(64, S - t * 64);
-        const float w = r < n ? pw[n - 1 - r] : 0.f;
+    auto store = [&](const Tile& x, int buf) {
 #pragma unroll
         for (int i = 0; i < 2; i++) {
-            u32x4 hi, lo, vv;
+            u32x4 hi, lo;
 #pragma unroll
             for (int e = 0; e < 4; e++) {
-                const float x0 = ((float)a[i][2 * e] + (float)b[i][2 * e]) * w, x1 = ((float)a[i][2 * e + 1] + (float)b[i][2 * e + 1]) * w;
+                const float x0 = ((float)x.a[i][2 * e] + (float)x.b[i][2 * e]) * x.w, x1 = ((float)x.a[i][2 * e + 1] + (float)x.b[i][2 * e + 1]) * x.w;
                 hi[e] = pack2(x0, x1);
                 lo[e] = pack2(x0 - lo16(hi[e]), x1 - hi16(hi[e]));
             }
-            vv = __builtin_bit_cast(u32x4, v[i]);
             const int at = r * 128 + (((c0 + i) ^ vswz<64>(r)) << 4);
-            *(u32x4*)(sm[buf][0] + at) = vv;
+            *(bf16x8*)(sm[buf][0] + at) = x.v[i];
             *(u32x4*)(sm[buf][1] + at) = hi;
             *(u32x4*)(sm[buf][2] + at) = lo;
         }
     };
     const int gq = lane >> 4, li = lane & 15, tq = li >> 2, tp = li & 3;
     const int lrow = 4 * hh + tq, clow = (gq & 1) * 2 + (tp >> 1), sw = vswz<64>(lrow), loff = lrow * 128 + (tp & 1) * 8;
-    const int nt = (S + 63) / 64;
-    load(0);
-    store(0, 0);
-    __syncthreads();
-    for (int t = 0; t < nt; t++) {
-        const int cur = t & 1;
-        if (t + 1 < nt) load(t + 1);
+    // tile t from LDS buffer `cur`; tile t + 1 goes from `x` to the other buffer, then tile t + 3 is requested into `x`
+    auto step = [&](int t, int cur, Tile& x) {
         if (t % (RET_CHUNK / 64) == 0) {
-            bf16* sn = p.snap + (((int64_t)(snap0 + t / (RET_CHUNK / 64)) * p.H + h) * 2 * p.Vp + dv0) * p.Kp + dk;
+            bf16* sn = p.snap + ((int64_t)(snap0 + t / (RET_CHUNK / 64)) * p.H + h) * 2 * p.Vp * p.Kp;
             const int64_t term = (int64_t)p.Vp * p.Kp;
 #pragma unroll
-            for (int e = 0; e < 16; e++) {
-                const int64_t o = ((e & 3) + 8 * (e >> 2)) * (int64_t)p.Kp;
-                const float hi = rbf(acc[e]);
-                sn[o] = f2bf(acc[e]);
-                sn[o + term] = f2bf(acc[e] - hi);
+            for (int g = 0; g < 4; g++) {
+                bf16x4 hi, lo;
+#pragma unroll
+                for (int e = 0; e < 4; e++) {
+                    const float v = acc[4 * g + e];
+                    hi[e] = f2bf(v);
+                    lo[e] = f2bf(v - rbf(v));
+                }
+                const int64_t o = ret_snap_at(dk0 + 8 * g, dv, p.Kp);
+                *(bf16x4*)(sn + o) = hi;
+                *(bf16x4*)(sn + term + o) = lo;
             }
         }
         const float w = pw[min(64, S - t * 64)];
@@ -232,14 +243,25 @@ __global__ __launch_bounds__(256) void ret_state_kernel(const RetParams p) {
             const bf16x8 vf = read_tr(sm[cur][0] + 16 * s * 128 + loff + ((((wv * 4) ^ sw) | clow) << 4), 128);
             const bf16x8 kf = read_tr(sm[cur][1] + 16 * s * 128 + loff + ((((wk * 4) ^ sw) | clow) << 4), 128);
             const bf16x8 kl = read_tr(sm[cur][2] + 16 * s * 128 + loff + ((((wk * 4) ^ sw) | clow) << 4), 128);
-            acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf, kf, acc, 0, 0, 0);
-            acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf, kl, acc, 0, 0, 0);
+            acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf, vf, acc, 0, 0, 0);
+            acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kl, vf, acc, 0, 0, 0);
         }
-        if (t + 1 < nt) store(t + 1, cur ^ 1);
+        if (t + 1 < nt) store(x, cur ^ 1);
+        if (t + 3 < nt) load(t + 3, x);
         __syncthreads();
+    };
+    Tile a, b;
+    load(0, a);
+    load(min(1, nt - 1), b);
+    store(a, 0);
+    load(min(2, nt - 1), a);
+    __syncthreads();
+    for (int t = 0; t < nt; t += 2) {
+        step(t, 0, b);
+        if (t + 1 < nt) step(t + 1, 1, a);
     }
 #pragma unroll
-    for (int e = 0; e < 16; e++) st[ret_state_at(dk, dv0 + (e & 3) + 8 * (e >> 2), NR)] = acc[e];
+    for (int e = 0; e < 16; e++) st[ret_state_at(dk0 + (e & 3) + 8 * (e >> 2), dv, NR)] = acc[e];
 }
 
 // 128 rows of one (segment, head): four waves of 32, key tiles of 32 rows from the chunk's start on (attention.hip's operand roles: queries on the lanes)
@@ -298,12 +320,12 @@ __global__ __launch_bounds__(256, (KP > 128 || VP > 128) ? 1 : 2) void ret_out_k
         for (int e = 0; e < 16; e++) oacc[db][e] = 0.f;
     __syncthreads();
     if ((chunk > 0 || sg[2] > 0) && w0 < S) {                 // what came before the chunk
-        const bf16* sn = p.snap + ((int64_t)(p.snap0[blockIdx.z] + chunk) * p.H + h) * 2 * VP * KP + (int64_t)l31 * KP + hh * 8;
+        const bf16* sn = p.snap + ((int64_t)(p.snap0[blockIdx.z] + chunk) * p.H + h) * 2 * VP * KP + lane * 8;
 #pragma unroll
         for (int db = 0; db < DB; db++)
 #pragma unroll
             for (int ks = 0; ks < KS; ks++) {
-                const bf16x8 sh = *(const bf16x8*)(sn + (int64_t)db * 32 * KP + ks * 16), sl = *(const bf16x8*)(sn + (int64_t)(VP + db * 32) * KP + ks * 16);
+                const bf16x8 sh = *(const bf16x8*)(sn + (db * KS + ks) * 512), sl = *(const bf16x8*)(sn + VP * KP + (db * KS + ks) * 512);
                 oacc[db] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(sh, qh[ks], oacc[db], 0, 0, 0);
                 oacc[db] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(sl, qh[ks], oacc[db], 0, 0, 0);
                 oacc[db] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(sh, ql[ks], oacc[db], 0, 0, 0);
@@ -412,18 +434,21 @@ int check(const char* who, const RetParams& p) {
     return CR_OK;
 }
 
-template <typename T>
-int decode_t(const RetParams& p, hipStream_t st) {
-    const dim3 grid(p.H, p.M);
-    const int blocks = p.Vp / 16;
-    switch (p.Kp) {
-        case 64: hipLaunchKernelGGL((ret_decode_kernel<T, 4>), grid, dim3(64 * min(blocks, dec_waves(4))), 0, st, p); break;
-        case 128: hipLaunchKernelGGL((ret_decode_kernel<T, 8>), grid, dim3(64 * min(blocks, dec_waves(8))), 0, st, p); break;
-        case 256: hipLaunchKernelGGL((ret_decode_kernel<T, 16>), grid, dim3(64 * min(blocks, dec_waves(16))), 0, st, p); break;
-        default: hipLaunchKernelGGL((ret_decode_kernel<T, 32>), grid, dim3(64 * min(blocks, dec_waves(32))), 0, st, p); break;
-    }
+template <typename T, int NR>
+int decode_n(const RetParams& p, const AttnParams* merge, int dim, hipStream_t st) {
+    const int waves = min(p.Vp / 16, dec_waves(NR)), extra = merge ? (merge->H * merge->Sq * (dim / 64) + waves - 1) / waves : 0;
+    hipLaunchKernelGGL((ret_decode_kernel<T, NR>), dim3(p.H + extra, p.M), dim3(64 * waves), 0, st, p, merge ? *merge : AttnParams{}, dim);
     CR_HIP(hipGetLastError());
     return CR_OK;
+}
+template <typename T>
+int decode_t(const RetParams& p, const AttnParams* merge, int dim, hipStream_t st) {
+    switch (p.Kp) {
+        case 64: return decode_n<T, 4>(p, merge, dim, st);
+        case 128: return decode_n<T, 8>(p, merge, dim, st);
+        case 256: return decode_n<T, 16>(p, merge, dim, st);
+    }
+    return decode_n<T, 32>(p, merge, dim, st);
 }
 
 template <typename T>
@@ -445,10 +470,12 @@ int recurrent_t(const RetParams& p, hipStream_t st) {
 
 bool ret_matrix_supported(int Kp, int Vp) { return Kp <= 256 && Vp <= 256; }
 
-int launch_ret_decode(bool f32, const RetParams& p, hipStream_t st) {
+int launch_ret_decode(bool f32, const RetParams& p, const AttnParams* merge, int merge_dim, hipStream_t st) {
     CR_TRY(check("retention (decode)", p));
     if (!p.rq || !p.rk || !p.ix.seqs || !p.ix.lens) return cr_fail(CR_ERR_ARG, "retention (decode): operands");
-    return f32 ? decode_t<float>(p, st) : decode_t<bf16>(p, st);
+    if (merge && (merge_dim <= 0 || merge_dim % 64 || merge->B != p.M || merge->H <= 0 || merge->Sq <= 0 || merge->nsplit <= 0 || !merge->part_o || !merge->part_ml || !merge->O))
+        return cr_fail(CR_ERR_ARG, "retention (decode): splits to merge");
+    return f32 ? decode_t<float>(p, merge, merge_dim, st) : decode_t<bf16>(p, merge, merge_dim, st);
 }
 
 int launch_ret_recurrent(bool f32, const RetParams& p, hipStream_t st) {
