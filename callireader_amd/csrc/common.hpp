@@ -166,12 +166,11 @@ enum GemmEpi {
     EPI_SWIGLU = 4,   // bf16(bf16(silu(bf16(g))) * bf16(u)), W rows interleaved [8 gate | 8 up]
     EPI_PATCH = 5,    // patch-embed: bf16(bf16(acc + bias) + pos[1 + m % G]) -> row (m / G) * (G + 1) + 1 + m % G
     EPI_F32 = 6,      // float(bf16(acc + bias))                            (logits: bf16 GEMM then .float())
-    EPI_PARTIAL = 7,  // decode only (M <= 64): fp32 partial sums [S][M][N] of S K-slices, no bias; the consumer kernel sums them
+    EPI_PARTIAL = 7,  // fp32 partial sums [S][M][N] of S K-slices, no bias; the consumer kernel sums them (M <= 64: S is the kernel's choice; 128-row kernel, kernel = 128: S = group)
     EPI_GELU_Q8 = 9,  // e4m3 instance only: e4m3(bf16(gelu(bf16(acc + bias))) / c8scale[m]) -- fc1's output as fc2's fp8 operand, no bf16 copy
     EPI_X_GLU = 10,   // grouped experts (gemm256 only): rows gathered through `perm`, W rows interleaved [8 gate | 8 up], clamped gated unit (GemmParams::limit)
     EPI_X_ROWS = 11,  // grouped experts (gemm256 only): plain rows, scattered through `perm`
     EPI_RELU2 = 12,   // bf16(max(acc, 0)^2), no bias
-    EPI_SIDE = 13,    // 128-row kernel only: bf16(gelu_tanh(acc) * res[perm[m]][n]): a gate times a row looked up by the token
     EPI_ARGMAX = 8,   // cosine VQ: C[m][b] = {col, bits(max)} of bf16(acc) over the 64 columns of block b (first max wins); nothing else stored
 };
 

@@ -40,6 +40,7 @@ __global__ __launch_bounds__(256, 2) void gemm128_kernel(const GemmParams p) {
     // ---- workgroup -> tile (XCD-aware, bijective for any grid size) ----
     const int ntm = (p.M + BM - 1) / BM, ntn = (p.N + BN - 1) / BN;
     const int nwg = gridDim.x, orig = blockIdx.x;
+    const int nk = p.K / BK / (int)gridDim.y;                 // K-tiles of this slice (EPI_PARTIAL: gridDim.y of them; one otherwise)
     const int xcd = orig & 7, q = nwg >> 3, r = nwg & 7;
     const int pid = (xcd < r ? xcd * (q + 1) : r * (q + 1) + (xcd - r) * q) + (orig >> 3);
     constexpr int GM = 8;
@@ -61,8 +62,8 @@ __global__ __launch_bounds__(256, 2) void gemm128_kernel(const GemmParams p) {
         const int ch = (lane & 7) ^ ((rr >> 1) & 7);
         const int gm = min(m0 + rr, p.M - 1);
         const int gn = min(n0 + rr, p.N - 1);
-        ga[i] = p.A + (int64_t)gm * p.lda + ch * 8;
-        gb[i] = p.W + (int64_t)gn * p.ldw + ch * 8;
+        ga[i] = p.A + (int64_t)gm * p.lda + ch * 8 + (int64_t)blockIdx.y * nk * BK;
+        gb[i] = p.W + (int64_t)gn * p.ldw + ch * 8 + (int64_t)blockIdx.y * nk * BK;
     }
     auto stage = [&](int buf, int kt) {
         char* base = smem + buf * 32768 + wave * 4096;
@@ -82,7 +83,6 @@ __global__ __launch_bounds__(256, 2) void gemm128_kernel(const GemmParams p) {
     const int swz = (lane >> 1) & 7;
     const int a_off = (wm * 64 + (lane & 15)) * 128;
     const int b_off = 16384 + (wn * 64 + (lane & 15)) * 128;
-    const int nk = p.K / BK;
 
     stage(0, 0);
     __syncthreads();
@@ -119,7 +119,11 @@ __global__ __launch_bounds__(256, 2) void gemm128_kernel(const GemmParams p) {
     __builtin_amdgcn_s_waitcnt(0xc07f);   // lgkmcnt(0): the stage is wave-private
     __builtin_amdgcn_wave_barrier();
 
-    epilogue_subtile<EPI>(p, st, m0 + wm * 64, n0 + wn * 64, lane);
+    if (EPI == EPI_PARTIAL) {
+        GemmParams q2 = p;
+        q2.C = (float*)p.C + (int64_t)blockIdx.y * p.M * p.ldc; q2.raw32 = 1; q2.softcap = 0.f;
+        epilogue_subtile<EPI_F32>(q2, st, m0 + wm * 64, n0 + wn * 64, lane);
+    } else epilogue_subtile<EPI == EPI_PARTIAL ? EPI_F32 : EPI>(p, st, m0 + wm * 64, n0 + wn * 64, lane);
 }
 
 template <int EPI>
@@ -127,7 +131,7 @@ int launch_t(const GemmParams& p, hipStream_t stream) {
     const int ntm = (p.M + BM - 1) / BM, ntn = (p.N + BN - 1) / BN;
     static std::atomic<uint64_t> attr_done{0};
     if (!cr_dyn_lds_once(attr_done, (const void*)gemm128_kernel<EPI>, LDS_BYTES)) return CR_ERR_HIP;
-    hipLaunchKernelGGL(gemm128_kernel<EPI>, dim3(ntm * ntn), dim3(256), LDS_BYTES, stream, p);
+    hipLaunchKernelGGL(gemm128_kernel<EPI>, dim3(ntm * ntn, EPI == EPI_PARTIAL ? p.group : 1), dim3(256), LDS_BYTES, stream, p);
     return hipGetLastError() == hipSuccess ? CR_OK : CR_ERR_HIP;
 }
 
@@ -186,7 +190,7 @@ int launch_gemm(int epi, const GemmParams& p, hipStream_t stream) {
         case EPI_STORE: return launch_t<EPI_STORE>(p, stream);
         case EPI_GELU: return launch_t<EPI_GELU>(p, stream);
         case EPI_RELU2: return launch_t<EPI_RELU2>(p, stream);
-        case EPI_SIDE: return (p.res && p.perm && (p.ldr & 7) == 0 && ((uintptr_t)p.res & 15) == 0 && p.N % 8 == 0) ? launch_t<EPI_SIDE>(p, stream) : CR_ERR_ARG;
+        case EPI_PARTIAL: return (!p.bias && p.group > 0 && p.K % (BK * p.group) == 0) ? launch_t<EPI_PARTIAL>(p, stream) : CR_ERR_ARG;
         case EPI_LS_RES: return (p.scale && p.res) ? launch_t<EPI_LS_RES>(p, stream) : CR_ERR_ARG;
         case EPI_RES: return p.res ? launch_t<EPI_RES>(p, stream) : CR_ERR_ARG;
         case EPI_SWIGLU: return (p.N % 16 == 0) ? launch_t<EPI_SWIGLU>(p, stream) : CR_ERR_ARG;

@@ -11,7 +11,7 @@ __device__ __forceinline__ void epilogue_row8(const GemmParams& p, int gm, int g
     // v[0..7]: fp32 accumulators of row gm, columns gn..gn+7 (gn % 8 == 0, gn + 8 <= N)
     float x[8];
     // EPI_STORE / EPI_PATCH-free paths whose only rounding is the final cast skip the explicit round-trip
-    constexpr bool ROUND_NOW = (EPI != EPI_STORE && EPI != EPI_F32 && EPI != EPI_RELU2 && EPI != EPI_SIDE);
+    constexpr bool ROUND_NOW = (EPI != EPI_STORE && EPI != EPI_F32 && EPI != EPI_RELU2);
     if (p.bias) {
         bf16x8 b = *(const bf16x8*)(p.bias + gn);
 #pragma unroll
@@ -37,10 +37,6 @@ __device__ __forceinline__ void epilogue_row8(const GemmParams& p, int gm, int g
     if (EPI == EPI_RELU2) {
 #pragma unroll
         for (int e = 0; e < 8; e++) x[e] = relu2(x[e]);
-    } else if (EPI == EPI_SIDE) {
-        const bf16x8 r = *(const bf16x8*)(p.res + (int64_t)p.perm[gm] * p.ldr + gn);
-#pragma unroll
-        for (int e = 0; e < 8; e++) x[e] = gelu_tanh(x[e]) * bf2f(r[e]);
     } else if (EPI == EPI_GELU) {
 #pragma unroll
         for (int e = 0; e < 8; e++) x[e] = gelu_erf(x[e]);
@@ -70,7 +66,7 @@ template <int EPI>
 __device__ __forceinline__ void epilogue_scalar(const GemmParams& p, int gm, int gn, float v) {
     const float sum = v + (p.bias ? bf2f(p.bias[gn]) : 0.0f);
     if (EPI == EPI_F32) { ((float*)p.C)[(int64_t)gm * p.ldc + gn] = f32_out(p, sum); return; }
-    float x = EPI == EPI_RELU2 ? relu2(sum) : EPI == EPI_SIDE ? gelu_tanh(sum) * bf2f(p.res[(int64_t)p.perm[gm] * p.ldr + gn]) : rbf(sum);
+    float x = EPI == EPI_RELU2 ? relu2(sum) : rbf(sum);
     int64_t orow = gm;
     if (EPI == EPI_GELU) x = gelu_erf(x);
     else if (EPI == EPI_LS_RES) x = bf2f(p.res[(int64_t)gm * p.ldr + gn]) + rbf(x * bf2f(p.scale[gn]));

@@ -246,7 +246,7 @@ struct Step {
     int nsplit, split;              // decode, latent attention: splits of the longest sequence, keys per split
     std::vector<KeyPlan> plans;     // prefill, one per distinct chunk size
     std::vector<int> hsplit;        // decode: attention splits per distinct chunk size
-    const int32_t *d_rseg, *d_snap0;      // prefill: {first row, rows, first position, sequence} per segment, its first state snapshot
+    const int32_t *d_rseg, *d_snap0, *d_chunks;      // prefill: {first row, rows, first position, sequence} per segment, its first retention chunk; {first row, rows} per chunk
     int snaps, longest;
 };
 
@@ -265,6 +265,25 @@ int heads_per_split(const cr_lm_heads& a) {
     while (n % d) d--;
     return d;
 }
+
+// decode of <= 64 rows: fp32 K-slices of A . W^T (gemm_skinny.hip) for a consumer that adds them; 0 when the shape has no such form.  Wide products of more than a few rows are one
+// slice through the kernel that splits N over its waves (gemm_stream.hip).
+GemmParams slice_params(const void* A, int64_t lda, const void* W, const bf16* dl, float* C, int M, int N, int K) {
+    GemmParams p{};
+    p.A = (const bf16*)A; p.lda = lda; p.W = dl ? dl : (const bf16*)W; p.ldw = K; p.wsw = dl ? 1 : 0; p.C = C; p.ldc = N; p.M = M; p.N = N; p.K = K;
+    return p;
+}
+bool one_slice(int M, int N, int K) { return gemm_stream_supported(EPI_F32, slice_params(nullptr, K, nullptr, nullptr, nullptr, M, N, K), 1); }
+int slices_of(const Lm& lm, int M, int N, int K, bool decode) { return lm.f32 || !decode || M > 64 ? 0 : one_slice(M, N, K) ? 1 : gemm_partial_splits(N, K); }
+int sliced(cr_ctx* c, const void* A, int64_t lda, const void* W, const bf16* dl, float* C, int M, int N, int K, hipStream_t st) {
+    GemmParams p = slice_params(A, lda, W, dl, C, M, N, K);
+    if (!one_slice(M, N, K)) return ctx_gemm(c, EPI_PARTIAL, p, st);
+    p.raw32 = 1;
+    return ctx_gemm(c, EPI_F32, p, st);
+}
+
+// K-slices of the token side's gate in the 128-row kernel: four where K allows (depends on K alone)
+int side_slices(int K) { return K % 256 == 0 ? 4 : K % 128 == 0 ? 2 : 1; }
 
 Buffers carve(const Lm& lm, Arena& ar, const Step& sp) {
     const size_t es = lm.esz();
@@ -300,7 +319,10 @@ Buffers carve(const Lm& lm, Arena& ar, const Step& sp) {
         Ep = std::max<size_t>(Ep, L.Ep); top = std::max<size_t>(top, L.s.top); act = std::max<size_t>(act, (size_t)L.s.top * L.ffp);
         tiles = std::max<size_t>(tiles, lm_max_tiles(M * L.s.top, L.s.experts, LM_TILE_M));
     }
-    if (lm.Sp) { slices(lm.Sp, Wp); slices(Wp, lm.Sp); }
+    if (lm.Sp) {
+        slices(lm.Sp, Wp); slices(Wp, lm.Sp);
+        if (!lm.f32 && !slices_of(lm, M, lm.Sp, Wp, decode)) sl = std::max(sl, (size_t)M * side_slices(Wp) * lm.Sp);
+    }
     if (lm.d.loop_in) slices(Wp, 2 * Wp);
     auto T = [&](size_t n) { return (void*)ar.take<char>(n * es); };
     Buffers b{};
@@ -318,22 +340,6 @@ size_t carve_bytes(const Lm& lm, const Step& sp) {
     Arena ar(nullptr);
     carve(lm, ar, sp);
     return ar.off + 512;
-}
-
-// decode of <= 64 rows: fp32 K-slices of A . W^T (gemm_skinny.hip) for a consumer that adds them; 0 when the shape has no such form.  Wide products of more than a few rows are one
-// slice through the kernel that splits N over its waves (gemm_stream.hip).
-GemmParams slice_params(const void* A, int64_t lda, const void* W, const bf16* dl, float* C, int M, int N, int K) {
-    GemmParams p{};
-    p.A = (const bf16*)A; p.lda = lda; p.W = dl ? dl : (const bf16*)W; p.ldw = K; p.wsw = dl ? 1 : 0; p.C = C; p.ldc = N; p.M = M; p.N = N; p.K = K;
-    return p;
-}
-bool one_slice(int M, int N, int K) { return gemm_stream_supported(EPI_F32, slice_params(nullptr, K, nullptr, nullptr, nullptr, M, N, K), 1); }
-int slices_of(const Lm& lm, int M, int N, int K, bool decode) { return lm.f32 || !decode || M > 64 ? 0 : one_slice(M, N, K) ? 1 : gemm_partial_splits(N, K); }
-int sliced(cr_ctx* c, const void* A, int64_t lda, const void* W, const bf16* dl, float* C, int M, int N, int K, hipStream_t st) {
-    GemmParams p = slice_params(A, lda, W, dl, C, M, N, K);
-    if (!one_slice(M, N, K)) return ctx_gemm(c, EPI_PARTIAL, p, st);
-    p.raw32 = 1;
-    return ctx_gemm(c, EPI_F32, p, st);
 }
 
 // C[M, N] = A . W^T in the model's element type: the engine's dense kernels for bf16, the fp32 tile kernel otherwise
@@ -472,7 +478,7 @@ int heads_mixer(cr_ctx* c, cr_kv* kv, const Step& sp, Buffers& b, const LmLayer&
     rp.rq = b.rq; rp.rk = b.rk; rp.rq2 = b.rq2; rp.rk2 = b.rk2; rp.lda = L.Na; rp.v = (char*)b.a + (size_t)L.region(LM_RV)->off * es; rp.g = (char*)b.a + (size_t)L.region(LM_RG)->off * es;
     rp.ao = (char*)b.ao + (size_t)L.off_r * es; rp.ldo = L.Gp; rp.state = (float*)(kv->lat + kv->state_off[r]); rp.raw = b.raw; rp.snap = b.snap; rp.pw = L.pw;
     rp.M = M; rp.H = rt.heads; rp.Kp = L.Kp; rp.Vp = L.Vp; rp.vdim = rt.vdim; rp.eps = lm.d.eps; rp.out_scale = rt.out_scale; rp.ix = sp.ix;
-    rp.seg = sp.d_rseg; rp.snap0 = sp.d_snap0; rp.n_segs = (int)sp.segs.size(); rp.longest = sp.longest;
+    rp.seg = sp.d_rseg; rp.snap0 = sp.d_snap0; rp.n_segs = (int)sp.segs.size(); rp.longest = sp.longest; rp.chunks = sp.d_chunks; rp.n_chunks = sp.snaps;
     return sp.decode ? launch_ret_decode(lm.f32, rp, merge ? &ap : nullptr, L.Ap, st) : matrix ? launch_ret_matrix(rp, st) : launch_ret_recurrent(lm.f32, rp, st);
 }
 
@@ -564,21 +570,22 @@ int run_passes(cr_ctx* c, cr_kv* kv, const Step& sp, Buffers& b, hipStream_t st)
             CR_TRY(launch_lm_post(lm.f32, lm, M, LmPostIn{b.ye, Wp, 0, b.wt, L.s.top}, b.x, L.n2b, false, end, st));
         }
         if (lm.Sp) {
-            const int n = slices_of(lm, M, lm.Sp, Wp, sp.decode);
             const char* side = (const char*)lm.side + (size_t)lm.passes[r] * lm.Sp * es;
             const int64_t lds = (int64_t)lm.layers.size() * lm.Sp;
-            if (n) {
-                CR_TRY(sliced(c, b.h, Wp, L.sgate, L.sgate_dl, b.sl, M, lm.Sp, Wp, st));
-                CR_TRY(launch_lm_side_act(lm, M, b.sl, n, side, lds, b.tok, b.z2, st));
-            } else if (!lm.f32) {
-                GemmParams g{};
-                g.A = (const bf16*)b.h; g.lda = Wp; g.W = (const bf16*)L.sgate; g.ldw = Wp; g.C = b.z2; g.ldc = lm.Sp; g.M = M; g.N = lm.Sp; g.K = Wp; g.kernel = 128;
-                g.res = (const bf16*)side; g.ldr = lds; g.perm = b.tok;
-                CR_TRY(ctx_gemm(c, EPI_SIDE, g, st));
-            } else {
+            if (lm.f32) {
                 LmGemmParams g{};
                 g.A = b.h; g.lda = Wp; g.W = L.sgate; g.ldw = Wp; g.C = b.z2; g.ldc = lm.Sp; g.M = M; g.N = lm.Sp; g.K = Wp; g.gate = side; g.ldg = lds; g.tok = b.tok;
-                CR_TRY(launch_lm_gemm(lm.f32, LM_SIDE, g, st));
+                CR_TRY(launch_lm_gemm(true, LM_SIDE, g, st));
+            } else {
+                // few columns: K-slices keep the chip busy, and the kernel that adds them applies the activation and the token's row
+                int n = slices_of(lm, M, lm.Sp, Wp, sp.decode);
+                if (n) CR_TRY(sliced(c, b.h, Wp, L.sgate, L.sgate_dl, b.sl, M, lm.Sp, Wp, st));
+                else {
+                    GemmParams g = slice_params(b.h, Wp, L.sgate, nullptr, b.sl, M, lm.Sp, Wp);
+                    g.kernel = 128; g.group = n = side_slices(Wp);
+                    CR_TRY(ctx_gemm(c, EPI_PARTIAL, g, st));
+                }
+                CR_TRY(launch_lm_side_act(lm, M, b.sl, n, side, lds, b.tok, b.z2, st));
             }
             CR_TRY(project(b.z2, L.sproj, L.sproj_dl, lm.Sp, y));
             CR_TRY(launch_lm_post(lm.f32, lm, M, y, b.x, L.ns, false, next, st));
@@ -837,7 +844,7 @@ int cr_llm_prefill_tokens(cr_ctx* c, cr_kv* kv, const int32_t* seqs, int n, cons
     CR_HIP(hipSetDevice(c->device));
     hipStream_t st = (hipStream_t)stream;
     const int V = lm.d.vocab, piece = std::max(n, std::min(std::max(n_want, 1), 4096));
-    // one host-to-device copy: tokens, then per row sequence and position, per segment its bounds (two orders), the last rows, first snapshots, the rows asked for, key plans
+    // one host-to-device copy: tokens, then per row sequence and position, per segment its bounds (two orders), the last rows, first retention chunks, the rows asked for, the chunks, key plans
     const size_t fixed = (size_t)M * 4 + (size_t)n * 10 + n_want;
     std::vector<int32_t> hv(fixed);
     memcpy(hv.data(), tokens, (size_t)M * 8);
@@ -850,10 +857,13 @@ int cr_llm_prefill_tokens(cr_ctx* c, cr_kv* kv, const int32_t* seqs, int n, cons
         memcpy(h_rseg + 4 * i, b1, 16);
         h_last[i] = sg.row0 + sg.S - 1;
         h_snap[i] = sp.snaps;
-        sp.snaps += ret_snapshots(sg.S);
+        sp.snaps += ret_chunks(sg.S);
         sp.longest = std::max(sp.longest, sg.S);
     }
     if (n_want) memcpy(h_want, want, (size_t)n_want * 4);
+    const size_t at_chunks = hv.size();
+    for (const Step::Seg& sg : sp.segs)
+        for (int t = 0; t < sg.S; t += RET_CHUNK) { hv.push_back(sg.row0 + t); hv.push_back(std::min(RET_CHUNK, sg.S - t)); }
     std::vector<KeyPlanAt> at;
     for (int chunk : lm.chunks) { at.push_back(plan_keys(sp, chunk, kv->max_tokens, hv)); sp.plans.push_back(at.back().k); }
     CR_TRY(ws_ensure(c, carve_bytes(lm, sp) + (size_t)piece * lm.Wp * lm.esz() + (size_t)n * V * 4 + hv.size() * 4 + 8192));
@@ -868,7 +878,7 @@ int cr_llm_prefill_tokens(cr_ctx* c, cr_kv* kv, const int32_t* seqs, int n, cons
     sp.tokens = (const int64_t*)dv;
     sp.ix.row_seq = dv + 2 * (size_t)M; sp.ix.row_pos = sp.ix.row_seq + M; sp.d_seg = sp.ix.row_pos + M; sp.d_rseg = sp.d_seg + 4 * n;
     const int32_t *d_last = sp.d_rseg + 4 * n, *d_want = d_last + 2 * n;
-    sp.d_snap0 = d_last + n;
+    sp.d_snap0 = d_last + n; sp.d_chunks = dv + at_chunks;
     for (size_t i = 0; i < at.size(); i++) {
         KeyPlan& k = sp.plans[i];
         k.row_key = dv + at[i].row_key; k.row_slot = dv + at[i].row_slot; k.pieces = dv + at[i].pieces; k.pre_key = dv + at[i].pre_key; k.pre_slot = dv + at[i].pre_slot;

@@ -205,15 +205,16 @@ struct RetParams {
     void* ao; int64_t ldo;                            // out: head h at column h * vdim
     float* state;                                     // this pass's states [n_seqs][heads][Vp * Kp]
     float* raw;                                       // prompts, recurrent form: [M][heads * Vp]
-    bf16* snap;                                       // prompts, matrix form: states ahead of every chunk [snapshots][heads][2][Vp][Kp], two bf16 terms
+    bf16* snap;                                       // prompts, matrix form: what every chunk adds, then the state ahead of it [chunks][heads][Vp * Kp * 4 bytes]
     const float* pw;                                  // [heads][RET_CHUNK + 1]
     int M, H, Kp, Vp, vdim;
     float eps, out_scale;
     LmRowIndex ix;
-    const int32_t* seg; const int32_t* snap0; int n_segs, longest;      // prompts: {first row, rows, first position, sequence} per segment, its first snapshot
+    const int32_t* seg; const int32_t* snap0; int n_segs, longest;      // prompts: {first row, rows, first position, sequence} per segment, its first chunk
+    const int32_t* chunks; int n_chunks;              // prompts, matrix form: {first row, rows} of every chunk of RET_CHUNK rows
 };
 bool ret_matrix_supported(int Kp, int Vp);
-inline int ret_snapshots(int rows) { return (rows + RET_CHUNK - 1) / RET_CHUNK; }
+inline int ret_chunks(int rows) { return (rows + RET_CHUNK - 1) / RET_CHUNK; }
 // merge: decode splits that the attention beside it left (AttnParams::no_merge), of heads of merge_dim columns
 int launch_ret_decode(bool f32, const RetParams& p, const AttnParams* merge, int merge_dim, hipStream_t st);
 int launch_ret_recurrent(bool f32, const RetParams& p, hipStream_t st);

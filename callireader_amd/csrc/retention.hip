@@ -4,12 +4,14 @@
 // (lm.hpp: 1 KiB per load instruction) that keeps the contraction over dk inside a wave.
 //
 // Prompts in bf16, matrix form: the sequence is cut into chunks of RET_CHUNK rows.  Within a chunk o_i = sum_j decay^(i-j) (q_i . k_j) v_j, what came before enters as
-// decay^(i+1) S^T q_i with S the state ahead of the chunk.  ret_state_kernel walks a sequence in tiles of 64 rows with a 64 x 64 block of S^T in accumulators and leaves the states
-// ahead of the chunks; ret_out_kernel then does all chunks at once.  Operands that are not bf16 by nature (rotated q and k, decayed k, states, decayed scores) enter the matrix
+// decay^(i+1) S^T q_i with S the state ahead of the chunk.  Three launches: ret_chunk_kernel forms what each chunk adds to the state, all chunks at once; ret_scan_kernel carries the
+// state through them (in place: a chunk's addition becomes the state ahead of it); ret_out_kernel computes the outputs, again all chunks at once.  Operands that are not bf16 by nature (rotated q and k, decayed k, states, decayed scores) enter the matrix
 // cores as two bf16 terms, value and remainder, products of two remainders left out: 2^-16 relative, against fp32's place in the recurrence.
 // Powers of the decay come from a table in fp32 made from double (decay^0 .. decay^RET_CHUNK): no logarithm, so decays of 0 and 1 are ordinary.
 //
 // Prompts in fp32, and sizes past the matrix form: the recurrence token by token, state in registers, then a norm-and-gate kernel.
+#include <algorithm>
+
 #include "attention_merge.hpp"
 #include "lm.hpp"
 
@@ -161,25 +163,23 @@ __device__ __forceinline__ bf16x8 read_tr(const char* at, int row_bytes) {
     return bf16x8{lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]};
 }
 
-// snapshot of a (chunk, head), two terms of [Vp / 32][Kp / 16] blocks of 1 KiB: S^T as ret_out_kernel's A operand (lane = value column % 32, + 32 for the second eight dk)
-__device__ __forceinline__ int64_t ret_snap_at(int dk, int dv, int Kp) { return ((int64_t)(dv >> 5) * (Kp >> 4) + (dk >> 4)) * 512 + ((dv & 31) + ((dk & 8) << 2)) * 8 + (dk & 7); }
+// A chunk's addition and the state ahead of it share the bytes of RetParams::snap: per (chunk, head) blocks of 32 value columns x 16 dk, 2 KiB each; lane = value column % 32 (+ 32 for
+// the second eight dk).  Addition: fp32, [dk % 8 / 4][lane][dk % 4].  State: two bf16 terms, [term][lane][dk % 8] -- ret_out_kernel's A operand, 1 KiB per load instruction.
 
-// S[64 dk][64 dv] of one (segment, head), 64 rows of the segment at a time: S <- decay^n S + (decay^(n-1-j) k_j)^T V.  Two tiles of loads are under way while one is multiplied.
-__global__ __launch_bounds__(256) void ret_state_kernel(const RetParams p) {
+// U[64 dk][64 dv] of one (chunk, head): sum over the chunk's n rows of decay^(n-1-j) k_j v_j^T.  Two tiles of 64 rows are under way while one is multiplied.
+__global__ __launch_bounds__(256) void ret_chunk_kernel(const RetParams p) {
     __shared__ __attribute__((aligned(16))) char sm[2][3][8192];          // [buffer][v, k, k's remainder][64 rows][64 columns]
     const int tid = threadIdx.x, lane = tid & 63;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int kt = blockIdx.x % (p.Kp / 64), vt = blockIdx.x / (p.Kp / 64), h = blockIdx.y;
-    const int32_t* sg = p.seg + 4 * blockIdx.z;
-    const int row0 = sg[0], S = sg[1], seq = sg[3], snap0 = p.snap0[blockIdx.z];
+    const int row0 = p.chunks[2 * blockIdx.z], S = p.chunks[2 * blockIdx.z + 1];
     const float* pw = p.pw + h * (RET_CHUNK + 1);
     const int64_t plane = (int64_t)p.M * p.H * p.Kp;
     const int l31 = lane & 31, hh = lane >> 5, wv = wave & 1, wk = wave >> 1;
-    float* st = p.state + ((int64_t)seq * p.H + h) * p.Vp * p.Kp;
-    const int NR = p.Kp / 16, dv = vt * 64 + wv * 32 + l31, dk0 = kt * 64 + wk * 32 + 4 * hh;      // lane: value column dv, element e: dk0 + (e & 3) + 8 (e >> 2)
-    f32x16 acc;
+    const int dv = vt * 64 + wv * 32 + l31, dk0 = kt * 64 + wk * 32 + 4 * hh;      // lane: value column dv, element e: dk0 + (e & 3) + 8 (e >> 2)
+    f32x16 acc[2];
 #pragma unroll
-    for (int e = 0; e < 16; e++) acc[e] = sg[2] == 0 ? 0.f : st[ret_state_at(dk0 + (e & 3) + 8 * (e >> 2), dv, NR)];
+    for (int e = 0; e < 16; e++) acc[0][e] = acc[1][e] = 0.f;
 
     // staging: a thread carries 16 columns of one row
     const int r = tid >> 2, c0 = (tid & 3) * 2;
@@ -188,14 +188,13 @@ __global__ __launch_bounds__(256) void ret_state_kernel(const RetParams p) {
     struct Tile { bf16x8 v[2], a[2], b[2]; float w; };
     const int nt = (S + 63) / 64;
     auto load = [&](int t, Tile& x) {
-        const int64_t q = min(t * 64 + r, S - 1);
-        const int n = min(64, S - t * 64);
-        x.w = r < n ? pw[n - 1 - r] : 0.f;
+        const int q = t * 64 + r, qc = min(q, S - 1);
+        x.w = q < S ? pw[S - 1 - qc] : 0.f;
 #pragma unroll
         for (int i = 0; i < 2; i++) {
-            x.v[i] = *(const bf16x8*)(vp + q * p.lda + i * 8);
-            x.a[i] = *(const bf16x8*)(kp + q * p.H * p.Kp + i * 8);
-            x.b[i] = *(const bf16x8*)(kp + plane + q * p.H * p.Kp + i * 8);
+            x.v[i] = *(const bf16x8*)(vp + (int64_t)qc * p.lda + i * 8);
+            x.a[i] = *(const bf16x8*)(kp + (int64_t)qc * p.H * p.Kp + i * 8);
+            x.b[i] = *(const bf16x8*)(kp + plane + (int64_t)qc * p.H * p.Kp + i * 8);
         }
     };
     auto store = [&](const Tile& x, int buf) {
@@ -218,33 +217,13 @@ __global__ __launch_bounds__(256) void ret_state_kernel(const RetParams p) {
     const int lrow = 4 * hh + tq, clow = (gq & 1) * 2 + (tp >> 1), sw = vswz<64>(lrow), loff = lrow * 128 + (tp & 1) * 8;
     // tile t from LDS buffer `cur`; tile t + 1 goes from `x` to the other buffer, then tile t + 3 is requested into `x`
     auto step = [&](int t, int cur, Tile& x) {
-        if (t % (RET_CHUNK / 64) == 0) {
-            bf16* sn = p.snap + ((int64_t)(snap0 + t / (RET_CHUNK / 64)) * p.H + h) * 2 * p.Vp * p.Kp;
-            const int64_t term = (int64_t)p.Vp * p.Kp;
-#pragma unroll
-            for (int g = 0; g < 4; g++) {
-                bf16x4 hi, lo;
-#pragma unroll
-                for (int e = 0; e < 4; e++) {
-                    const float v = acc[4 * g + e];
-                    hi[e] = f2bf(v);
-                    lo[e] = f2bf(v - rbf(v));
-                }
-                const int64_t o = ret_snap_at(dk0 + 8 * g, dv, p.Kp);
-                *(bf16x4*)(sn + o) = hi;
-                *(bf16x4*)(sn + term + o) = lo;
-            }
-        }
-        const float w = pw[min(64, S - t * 64)];
-#pragma unroll
-        for (int e = 0; e < 16; e++) acc[e] *= w;
 #pragma unroll
         for (int s = 0; s < 4; s++) {
             const bf16x8 vf = read_tr(sm[cur][0] + 16 * s * 128 + loff + ((((wv * 4) ^ sw) | clow) << 4), 128);
             const bf16x8 kf = read_tr(sm[cur][1] + 16 * s * 128 + loff + ((((wk * 4) ^ sw) | clow) << 4), 128);
             const bf16x8 kl = read_tr(sm[cur][2] + 16 * s * 128 + loff + ((((wk * 4) ^ sw) | clow) << 4), 128);
-            acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf, vf, acc, 0, 0, 0);
-            acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kl, vf, acc, 0, 0, 0);
+            acc[0] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf, vf, acc[0], 0, 0, 0);
+            acc[1] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kl, vf, acc[1], 0, 0, 0);
         }
         if (t + 1 < nt) store(x, cur ^ 1);
         if (t + 3 < nt) load(t + 3, x);
@@ -260,17 +239,66 @@ __global__ __launch_bounds__(256) void ret_state_kernel(const RetParams p) {
         step(t, 0, b);
         if (t + 1 < nt) step(t + 1, 1, a);
     }
+    float* u = (float*)p.snap + ((int64_t)blockIdx.z * p.H + h) * p.Vp * p.Kp;
 #pragma unroll
-    for (int e = 0; e < 16; e++) st[ret_state_at(dk0 + (e & 3) + 8 * (e >> 2), dv, NR)] = acc[e];
+    for (int g = 0; g < 4; g++) {
+        const int dk = dk0 + 8 * g;
+        f32x4 o;
+#pragma unroll
+        for (int e = 0; e < 4; e++) o[e] = acc[0][4 * g + e] + acc[1][4 * g + e];
+        *(f32x4*)(u + ((int64_t)(dv >> 5) * (p.Kp >> 4) + (dk >> 4)) * 512 + hh * 256 + ((dv & 31) + ((dk & 8) << 2)) * 4) = o;
+    }
 }
 
-// 128 rows of one (segment, head): four waves of 32, key tiles of 32 rows from the chunk's start on (attention.hip's operand roles: queries on the lanes)
+// the state of one (segment, head) through its chunks, eight dk of one value column per thread; what a thread reads of a chunk it overwrites with the state ahead of it
+__global__ __launch_bounds__(256) void ret_scan_kernel(const RetParams p) {
+    const int t = blockIdx.x * 256 + threadIdx.x, h = blockIdx.y, lane = t & 63, blk = t >> 6, NR = p.Kp >> 4;
+    if (t * 8 >= p.Vp * p.Kp) return;
+    const int32_t* sg = p.seg + 4 * blockIdx.z;
+    const int n = (sg[1] + RET_CHUNK - 1) / RET_CHUNK, dv = blk / NR * 32 + (lane & 31), dk = blk % NR * 16 + (lane >> 5) * 8;
+    const float* pw = p.pw + h * (RET_CHUNK + 1);
+    float* st = p.state + ((int64_t)sg[3] * p.H + h) * p.Vp * p.Kp;
+    float* u = (float*)p.snap + ((int64_t)p.snap0[blockIdx.z] * p.H + h) * p.Vp * p.Kp + (int64_t)blk * 512 + lane * 4;
+    const int64_t step = (int64_t)p.H * p.Vp * p.Kp;
+    float s[8];
+#pragma unroll
+    for (int e = 0; e < 8; e++) s[e] = sg[2] == 0 ? 0.f : st[ret_state_at(dk + e, dv, NR)];
+    f32x4 a = *(const f32x4*)u, b = *(const f32x4*)(u + 256);
+    for (int c = 0; c < n; c++) {
+        const f32x4 na = *(const f32x4*)(u + min(c + 1, n - 1) * step), nb = *(const f32x4*)(u + min(c + 1, n - 1) * step + 256);
+        const float w = pw[min(RET_CHUNK, sg[1] - c * RET_CHUNK)];
+        bf16x8 hi, lo;
+#pragma unroll
+        for (int e = 0; e < 8; e++) {
+            hi[e] = f2bf(s[e]);
+            lo[e] = f2bf(s[e] - rbf(s[e]));
+            s[e] = s[e] * w + (e < 4 ? a[e] : b[e - 4]);
+        }
+        *(bf16x8*)(u + c * step) = hi;
+        *(bf16x8*)(u + c * step + 256) = lo;
+        a = na; b = nb;
+    }
+#pragma unroll
+    for (int e = 0; e < 8; e++) st[ret_state_at(dk + e, dv, NR)] = s[e];
+}
+
+// LDS-DMA from inline asm (M0 = LDS base, saved and restored inside the statement): the compiler does not order a tile's LDS reads behind the fills of later tiles
+__device__ __forceinline__ void dma16(const void* base, unsigned off, unsigned dst) {
+    unsigned keep;
+    asm volatile("s_mov_b32 %0, m0\n\ts_mov_b32 m0, %3\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, %2\n\ts_mov_b32 m0, %0" : "=&s"(keep) : "v"(off), "s"(base), "s"(dst) : "memory");
+}
+// all but the last N of this wave's loads have landed, for every wave of the workgroup
+template <int N> __device__ __forceinline__ void tile_barrier() { asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)\n\ts_barrier" ::"n"(N) : "memory"); }
+
+// 128 rows of one (segment, head): four waves of 32 (attention.hip's operand roles: queries on the lanes).  One stream of tiles through a ring of three LDS buffers, two under way:
+// the state ahead of the chunk in tiles of 32 value columns (what they give is exactly their block of the output), then the chunk's keys and values in tiles of 32 rows.
 template <int KP, int VP>
 __global__ __launch_bounds__(256, (KP > 128 || VP > 128) ? 1 : 2) void ret_out_kernel(const RetParams p) {
     extern __shared__ __attribute__((aligned(16))) char smem[];
     constexpr int KB = 32 * KP * 2, VB = 32 * VP * 2, BUF = 2 * KB + VB;
     constexpr int KS = KP / 16, DB = VP / 32;
-    float* pwl = (float*)(smem + 2 * BUF);                    // [RET_CHUNK + 1]
+    constexpr int NK = KB / 4096, NV = VB / 4096, NTILE = 2 * NK + NV, NSTATE = 2 * NK;      // load instructions per wave: keys (one term), values, a tile, a state tile
+    float* pwl = (float*)(smem + 3 * BUF);                    // 32 zeros, then decay^0 .. decay^RET_CHUNK: a key behind its query weighs nothing
     const int tid = threadIdx.x, lane = tid & 63;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int l31 = lane & 31, hh = lane >> 5;
@@ -281,31 +309,44 @@ __global__ __launch_bounds__(256, (KP > 128 || VP > 128) ? 1 : 2) void ret_out_k
     const int chunk = blk / (RET_CHUNK / 128), c0 = chunk * RET_CHUNK;
     const int w0 = blk * 128 + wave * 32, qi = w0 + l31, qc = min(qi, S - 1);
     const int64_t plane = (int64_t)p.M * p.H * KP;
-    for (int i = tid; i <= RET_CHUNK; i += 256) pwl[i] = p.pw[h * (RET_CHUNK + 1) + i];
+    const bool prior = chunk > 0 || sg[2] > 0;
 
     const bf16* kb = p.rk2 + ((int64_t)(row0 + c0) * p.H + h) * KP;
     const bf16* vb = (const bf16*)p.v + (int64_t)(row0 + c0) * p.lda + h * VP;
+    const bf16* sn = p.snap + ((int64_t)(p.snap0[blockIdx.z] + chunk) * p.H + h) * 2 * VP * KP;
     const int last = S - 1 - c0;                              // last row of the segment, counted from the chunk
-    auto stage = [&](int buf, int kt) {
-        constexpr int KR = 1024 / (KP * 2), VR = 1024 / (VP * 2);         // rows per load instruction
-        char* base = smem + buf * BUF;
+    const unsigned lds = (unsigned)(size_t)(__attribute__((address_space(3))) char*)smem;
+    const int ns = prior ? DB : 0, nt = (min(blk * 128 + 128, S) - c0 + 31) / 32;
+    // tile u of the stream: a state tile (u < ns), else keys and values; chunks of 16 bytes swizzled on the source side
+    auto stage = [&](int buf, int u) {
+        const unsigned base = lds + buf * BUF;
+        if (u < ns) {
 #pragma unroll
-        for (int i = 0; i < 32 / KR / 4; i++) {
-            const int r = (wave * (32 / KR / 4) + i) * KR + lane / (KP / 8), cp = lane % (KP / 8);
-            const bf16* s = kb + (int64_t)min(kt * 32 + r, last) * p.H * KP + ((cp ^ kswz<KP>(r)) * 8);
-            char* d = base + (wave * (32 / KR / 4) + i) * 1024;
-            __builtin_amdgcn_global_load_lds(CR_GLB(s), CR_LDS(d), 16, 0, 0);
-            __builtin_amdgcn_global_load_lds(CR_GLB(s + plane), CR_LDS(d + KB), 16, 0, 0);
+            for (int i = 0; i < NSTATE; i++) dma16(sn, (unsigned)(u * 2 * KB + (wave * NSTATE + i) * 1024 + lane * 16), base + (wave * NSTATE + i) * 1024);
+            return;
+        }
+        constexpr int KR = 1024 / (KP * 2), VR = 1024 / (VP * 2);         // rows per load instruction
+        const int key = (u - ns) * 32;
+#pragma unroll
+        for (int i = 0; i < NK; i++) {
+            const int r = (wave * NK + i) * KR + lane / (KP / 8), cp = lane % (KP / 8);
+            const unsigned off = (unsigned)min(key + r, last) * (unsigned)(p.H * KP * 2) + (unsigned)((cp ^ kswz<KP>(r)) * 16);
+            dma16(kb, off, base + (wave * NK + i) * 1024);
+            dma16(kb + plane, off, base + KB + (wave * NK + i) * 1024);
         }
 #pragma unroll
-        for (int i = 0; i < 32 / VR / 4; i++) {
-            const int r = (wave * (32 / VR / 4) + i) * VR + lane / (VP / 8), cp = lane % (VP / 8);
-            const bf16* s = vb + (int64_t)min(kt * 32 + r, last) * p.lda + ((cp ^ vswz<VP>(r)) * 8);
-            __builtin_amdgcn_global_load_lds(CR_GLB(s), CR_LDS(base + 2 * KB + (wave * (32 / VR / 4) + i) * 1024), 16, 0, 0);
+        for (int i = 0; i < NV; i++) {
+            const int r = (wave * NV + i) * VR + lane / (VP / 8), cp = lane % (VP / 8);
+            dma16(vb, (unsigned)min(key + r, last) * (unsigned)(p.lda * 2) + (unsigned)((cp ^ vswz<VP>(r)) * 16), base + 2 * KB + (wave * NV + i) * 1024);
         }
     };
-    const int nt = (min(blk * 128 + 128, S) - c0 + 31) / 32;
-    stage(0, 0);
+    const int total = ns + nt;
+    // behind tile u: tile u + 1 has landed, tile u + 2 may be under way
+    auto close = [&](int u) {
+        if (u + 2 >= total) tile_barrier<0>();
+        else if (u + 2 < ns) tile_barrier<NSTATE>();
+        else tile_barrier<NTILE>();
+    };
 
     bf16x8 qh[KS], ql[KS];
     {
@@ -313,24 +354,36 @@ __global__ __launch_bounds__(256, (KP > 128 || VP > 128) ? 1 : 2) void ret_out_k
 #pragma unroll
         for (int ks = 0; ks < KS; ks++) { qh[ks] = *(const bf16x8*)(q + ks * 16); ql[ks] = *(const bf16x8*)(q + plane + ks * 16); }
     }
+    for (int i = tid; i < RET_CHUNK + 33; i += 256) pwl[i] = i < 32 ? 0.f : p.pw[h * (RET_CHUNK + 1) + i - 32];
+    __builtin_amdgcn_s_waitcnt(0x0F70);       // vmcnt(0) the compiler sees: without it the queries' first use waits for the fills below
+    stage(0, 0);
+    if (total > 1) stage(1, 1);
     f32x16 oacc[DB];
 #pragma unroll
     for (int db = 0; db < DB; db++)
 #pragma unroll
         for (int e = 0; e < 16; e++) oacc[db][e] = 0.f;
-    __syncthreads();
-    if ((chunk > 0 || sg[2] > 0) && w0 < S) {                 // what came before the chunk
-        const bf16* sn = p.snap + ((int64_t)(p.snap0[blockIdx.z] + chunk) * p.H + h) * 2 * VP * KP + lane * 8;
+    close(-1);
+    int slot = 0;                                             // ring place of the current tile
+    auto ring = [](int i) { return i >= 3 ? i - 3 : i; };
+    if (prior) {                                              // what came before the chunk
 #pragma unroll
-        for (int db = 0; db < DB; db++)
+        for (int db = 0; db < DB; db++) {
+            if (db + 2 < total) stage(ring(slot + 2), db + 2);
+            if (w0 < S) {
+                const char* base = smem + slot * BUF + lane * 16;
 #pragma unroll
-            for (int ks = 0; ks < KS; ks++) {
-                const bf16x8 sh = *(const bf16x8*)(sn + (db * KS + ks) * 512), sl = *(const bf16x8*)(sn + VP * KP + (db * KS + ks) * 512);
-                oacc[db] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(sh, qh[ks], oacc[db], 0, 0, 0);
-                oacc[db] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(sl, qh[ks], oacc[db], 0, 0, 0);
-                oacc[db] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(sh, ql[ks], oacc[db], 0, 0, 0);
+                for (int ks = 0; ks < KS; ks++) {
+                    const bf16x8 sh = *(const bf16x8*)(base + ks * 2048), sl = *(const bf16x8*)(base + ks * 2048 + 1024);
+                    oacc[db] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(sh, qh[ks], oacc[db], 0, 0, 0);
+                    oacc[db] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(sl, qh[ks], oacc[db], 0, 0, 0);
+                    oacc[db] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(sh, ql[ks], oacc[db], 0, 0, 0);
+                }
             }
-        const float w = pwl[qc - c0 + 1];
+            close(db);
+            slot = ring(slot + 1);
+        }
+        const float w = pwl[32 + qc - c0 + 1];
 #pragma unroll
         for (int db = 0; db < DB; db++)
 #pragma unroll
@@ -341,10 +394,10 @@ __global__ __launch_bounds__(256, (KP > 128 || VP > 128) ? 1 : 2) void ret_out_k
     const int gq = lane >> 4, li = lane & 15, tq = li >> 2, tp = li & 3;
     const int v_row = 4 * hh + tq, v_sw = vswz<VP>(v_row), v_clow = (gq & 1) * 2 + (tp >> 1), v_off = v_row * VP * 2 + (tp & 1) * 8;
     for (int kt = 0; kt < nt; kt++) {
-        const int cur = kt & 1, key0 = c0 + kt * 32;
-        if (kt + 1 < nt) stage(cur ^ 1, kt + 1);
-        const char* base = smem + cur * BUF;
-        if (w0 < S && key0 <= w0 + 31) {
+        const int key0 = c0 + kt * 32, u = ns + kt;
+        if (u + 2 < total) stage(ring(slot + 2), u + 2);
+        const char* base = smem + slot * BUF;
+        if (w0 < S && key0 <= w0) {                           // (tiles and waves both start at multiples of 32: a later tile is all behind the wave's queries)
             f32x16 s;
 #pragma unroll
             for (int e = 0; e < 16; e++) s[e] = 0.f;
@@ -357,11 +410,11 @@ __global__ __launch_bounds__(256, (KP > 128 || VP > 128) ? 1 : 2) void ret_out_k
                 s = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf, ql[ks], s, 0, 0, 0);
             }
             unsigned ph[8], pl[8];
-            const int d0 = qc - key0 - 4 * hh;                // rows between the query and the lane's first key
+            const float* wl = pwl + 32 + qc - key0 - 4 * hh;  // decay of the lane's first key
 #pragma unroll
             for (int i = 0; i < 8; i++) {
-                const int e = 2 * i, d = d0 - ((e & 3) + 8 * (e >> 2));
-                const float x0 = s[e] * (d >= 0 ? pwl[max(d, 0)] : 0.f), x1 = s[e + 1] * (d >= 1 ? pwl[max(d - 1, 0)] : 0.f);
+                const int e = 2 * i, k = (e & 3) + 8 * (e >> 2);
+                const float x0 = s[e] * wl[-k], x1 = s[e + 1] * wl[-k - 1];
                 ph[i] = pack2(x0, x1);
                 pl[i] = pack2(x0 - lo16(ph[i]), x1 - hi16(ph[i]));
             }
@@ -377,7 +430,8 @@ __global__ __launch_bounds__(256, (KP > 128 || VP > 128) ? 1 : 2) void ret_out_k
                 }
             }
         }
-        __syncthreads();
+        close(u);
+        slot = ring(slot + 1);
     }
 
     // ---- norm over the head, gate, store: lane (query, half) owns d = 32 db + 8 g4 + 4 hh + 0..3 ----
@@ -411,7 +465,7 @@ __global__ __launch_bounds__(256, (KP > 128 || VP > 128) ? 1 : 2) void ret_out_k
 
 template <int KP, int VP>
 int launch_out(const RetParams& p, hipStream_t st) {
-    constexpr int LDS = 2 * 32 * 2 * (2 * KP + VP) + (RET_CHUNK + 4) * 4;
+    constexpr int LDS = 3 * 32 * 2 * (2 * KP + VP) + (RET_CHUNK + 36) * 4;
     static std::atomic<uint64_t> attr_done{0};
     if (!cr_dyn_lds_once(attr_done, (const void*)ret_out_kernel<KP, VP>, LDS)) return cr_fail(CR_ERR_HIP, "retention: LDS");
     hipLaunchKernelGGL((ret_out_kernel<KP, VP>), dim3((p.longest + 127) / 128, p.H, p.n_segs), dim3(256), LDS, st, p);
@@ -486,8 +540,15 @@ int launch_ret_recurrent(bool f32, const RetParams& p, hipStream_t st) {
 
 int launch_ret_matrix(const RetParams& p, hipStream_t st) {
     CR_TRY(check("retention (matrix)", p));
-    if (!ret_matrix_supported(p.Kp, p.Vp) || !p.rq2 || !p.rk2 || !p.snap || !p.seg || !p.snap0 || p.n_segs <= 0 || p.longest <= 0) return cr_fail(CR_ERR_ARG, "retention (matrix): operands");
-    hipLaunchKernelGGL(ret_state_kernel, dim3(p.Kp / 64 * (p.Vp / 64), p.H, p.n_segs), dim3(256), 0, st, p);
+    if (!ret_matrix_supported(p.Kp, p.Vp) || !p.rq2 || !p.rk2 || !p.snap || !p.seg || !p.snap0 || !p.chunks || p.n_chunks <= 0 || p.n_segs <= 0 || p.longest <= 0 || p.n_segs > 65535 ||
+        (int64_t)RET_CHUNK * std::max<int64_t>(p.lda * 2, (int64_t)p.H * p.Kp * 2) >= (1ll << 31)) return cr_fail(CR_ERR_ARG, "retention (matrix): operands");
+    for (int i = 0; i < p.n_chunks; i += 32768) {             // (a grid's third dimension)
+        RetParams q = p;
+        q.chunks += 2 * (size_t)i; q.snap += (int64_t)i * p.H * 2 * p.Vp * p.Kp;
+        hipLaunchKernelGGL(ret_chunk_kernel, dim3(p.Kp / 64 * (p.Vp / 64), p.H, min(32768, p.n_chunks - i)), dim3(256), 0, st, q);
+        CR_HIP(hipGetLastError());
+    }
+    hipLaunchKernelGGL(ret_scan_kernel, dim3((p.Vp * p.Kp / 8 + 255) / 256, p.H, p.n_segs), dim3(256), 0, st, p);
     CR_HIP(hipGetLastError());
     switch (p.Kp) {
         case 64: return launch_out_k<64>(p, st);
