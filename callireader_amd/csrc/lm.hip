@@ -519,7 +519,8 @@ int expert_mixture(cr_ctx* c, const Step& sp, Buffers& b, const LmLayer& L, hipS
     return CR_OK;
 }
 
-int run_passes(cr_ctx* c, cr_kv* kv, const Step& sp, Buffers& b, hipStream_t st) {
+// last: where the final norm of every row goes (decode); null: the residual stays in b.x, rows are picked from it afterwards
+int run_passes(cr_ctx* c, cr_kv* kv, const Step& sp, Buffers& b, void* last, hipStream_t st) {
     const Lm& lm = *c->lm;
     const int M = sp.M, Wp = lm.Wp;
     const size_t es = lm.esz();
@@ -531,7 +532,7 @@ int run_passes(cr_ctx* c, cr_kv* kv, const Step& sp, Buffers& b, hipStream_t st)
     };
     // what reads the residual ahead of pass r: its first norm, or the product that mixes the embedding in
     auto entry = [&](size_t r) -> LmSink {
-        if (r >= lm.passes.size()) return {nullptr, 0, nullptr};
+        if (r >= lm.passes.size()) return {last, Wp, lm.fin};
         if (lm.starts[r]) return {b.cat, 2 * Wp, nullptr};
         return {b.h, Wp, lm.layers[lm.passes[r]].n1};
     };
@@ -572,6 +573,7 @@ int run_passes(cr_ctx* c, cr_kv* kv, const Step& sp, Buffers& b, hipStream_t st)
         if (lm.Sp) {
             const char* side = (const char*)lm.side + (size_t)lm.passes[r] * lm.Sp * es;
             const int64_t lds = (int64_t)lm.layers.size() * lm.Sp;
+            bool projected = false;
             if (lm.f32) {
                 LmGemmParams g{};
                 g.A = b.h; g.lda = Wp; g.W = L.sgate; g.ldw = Wp; g.C = b.z2; g.ldc = lm.Sp; g.M = M; g.N = lm.Sp; g.K = Wp; g.gate = side; g.ldg = lds; g.tok = b.tok;
@@ -585,9 +587,12 @@ int run_passes(cr_ctx* c, cr_kv* kv, const Step& sp, Buffers& b, hipStream_t st)
                     g.kernel = 128; g.group = n = side_slices(Wp);
                     CR_TRY(ctx_gemm(c, EPI_PARTIAL, g, st));
                 }
-                CR_TRY(launch_lm_side_act(lm, M, b.sl, n, side, lds, b.tok, b.z2, st));
+                projected = sp.decode && lm_side_proj_supported(lm, M);
+                if (projected) CR_TRY(launch_lm_side_proj(lm, M, b.sl, n, side, lds, b.tok, L.sproj, b.y, st));
+                else CR_TRY(launch_lm_side_act(lm, M, b.sl, n, side, lds, b.tok, b.z2, st));
             }
-            CR_TRY(project(b.z2, L.sproj, L.sproj_dl, lm.Sp, y));
+            if (projected) y = LmPostIn{b.y, Wp, 0, nullptr, 0};
+            else CR_TRY(project(b.z2, L.sproj, L.sproj_dl, lm.Sp, y));
             CR_TRY(launch_lm_post(lm.f32, lm, M, y, b.x, L.ns, false, next, st));
         }
         CR_TRY(probe((int)r + 1));
@@ -595,12 +600,12 @@ int run_passes(cr_ctx* c, cr_kv* kv, const Step& sp, Buffers& b, hipStream_t st)
     return CR_OK;
 }
 
-// final norm of n rows of x (rows: device indices, null = 0 .. n), then the logits, in pieces that fit `hl`
-int lm_head(cr_ctx* c, const Lm& lm, const float* x, const int32_t* rows, int n, void* hl, int piece, float* out, hipStream_t st, bool decode) {
+// final norm of n rows of x (device indices), then the logits, in pieces that fit `hl`
+int lm_head(cr_ctx* c, const Lm& lm, const float* x, const int32_t* rows, int n, void* hl, int piece, float* out, hipStream_t st) {
     for (int i = 0; i < n; i += piece) {
         const int m = std::min(piece, n - i);
-        CR_TRY(launch_lm_pick_rows(lm.f32, lm, m, rows ? x : x + (size_t)i * lm.Wp, rows ? rows + i : nullptr, hl, lm.fin, st));
-        CR_TRY(raw32(c, lm, hl, lm.head, out + (size_t)i * lm.d.vocab, lm.d.vocab, m, lm.d.vocab, lm.Wp, lm.d.softcap, st, decode ? lm.head_dl : nullptr));
+        CR_TRY(launch_lm_pick_rows(lm.f32, lm, m, x, rows + i, hl, lm.fin, st));
+        CR_TRY(raw32(c, lm, hl, lm.head, out + (size_t)i * lm.d.vocab, lm.d.vocab, m, lm.d.vocab, lm.Wp, lm.d.softcap, st));
     }
     return CR_OK;
 }
@@ -692,8 +697,8 @@ int lm_decode_step(cr_ctx* c, cr_kv* kv, int n, const int64_t* force_tokens, flo
     Buffers b = carve(lm, ar, sp);
     void* hl = ar.take<char>((size_t)n * lm.Wp * lm.esz());
     float* lg = ar.take<float>((size_t)n * lm.d.vocab);
-    CR_TRY(run_passes(c, kv, sp, b, st));
-    CR_TRY(lm_head(c, lm, b.x, nullptr, n, hl, n, lg, st, true));
+    CR_TRY(run_passes(c, kv, sp, b, hl, st));
+    CR_TRY(raw32(c, lm, hl, lm.head, lg, lm.d.vocab, n, lm.d.vocab, lm.Wp, lm.d.softcap, st, lm.head_dl));
     if (logits) CR_HIP(hipMemcpyAsync(logits, lg, (size_t)n * lm.d.vocab * 4, hipMemcpyDeviceToDevice, st));
     return launch_pick(lg, lm.d.vocab, lm.d.vocab, penalty, n, kv->d_seqs, kv, 1, st);
 }
@@ -883,9 +888,9 @@ int cr_llm_prefill_tokens(cr_ctx* c, cr_kv* kv, const int32_t* seqs, int n, cons
         KeyPlan& k = sp.plans[i];
         k.row_key = dv + at[i].row_key; k.row_slot = dv + at[i].row_slot; k.pieces = dv + at[i].pieces; k.pre_key = dv + at[i].pre_key; k.pre_slot = dv + at[i].pre_slot;
     }
-    CR_TRY(run_passes(c, kv, sp, b, st));
-    if (n_want) CR_TRY(lm_head(c, lm, b.x, d_want, n_want, hl, piece, want_logits, st, false));
-    CR_TRY(lm_head(c, lm, b.x, d_last, n, hl, piece, lg, st, false));
+    CR_TRY(run_passes(c, kv, sp, b, nullptr, st));
+    if (n_want) CR_TRY(lm_head(c, lm, b.x, d_want, n_want, hl, piece, want_logits, st));
+    CR_TRY(lm_head(c, lm, b.x, d_last, n, hl, piece, lg, st));
     if (last_logits) CR_HIP(hipMemcpyAsync(last_logits, lg, (size_t)n * V * 4, hipMemcpyDeviceToDevice, st));
     CR_TRY(launch_pick(lg, V, V, penalty, n, kv->d_seqs, kv, 0, st));
     for (const Step::Seg& sg : sp.segs) {

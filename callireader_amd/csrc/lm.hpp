@@ -221,6 +221,9 @@ int launch_ret_recurrent(bool f32, const RetParams& p, hipStream_t st);
 int launch_ret_matrix(const RetParams& p, hipStream_t st);
 // decode of <= 64 rows: z[m][n] = gelu_tanh(sum of K-slices) * side[tok[m]][n]
 int launch_lm_side_act(const Lm& lm, int M, const float* part, int slices, const void* side, int64_t lds, const int32_t* tok, void* z, hipStream_t st);
+// ... and y [M][Wp] = z . W^T in the same launch (few rows)
+bool lm_side_proj_supported(const Lm& lm, int M);
+int launch_lm_side_proj(const Lm& lm, int M, const float* part, int slices, const void* side, int64_t lds, const int32_t* tok, const void* W, void* y, hipStream_t st);
 
 int lm_finalize(cr_ctx* c, hipStream_t st);
 struct cr_kv;

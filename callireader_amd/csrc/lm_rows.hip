@@ -286,10 +286,62 @@ __global__ __launch_bounds__(256) void lm_side_act_kernel(const float* __restric
     const f32x4 e = ld4(side + (int64_t)tok[m] * lds + n);
     st4(z + i, f32x4{gelu_tanh(s[0]) * e[0], gelu_tanh(s[1]) * e[1], gelu_tanh(s[2]) * e[2], gelu_tanh(s[3]) * e[3]});
 }
+
+// the same z for up to 16 rows, kept in LDS, and y = z . W^T behind it: a workgroup forms z for itself (a few KiB from L2) and multiplies 64 rows of W, 16 per wave
+__global__ __launch_bounds__(256) void lm_side_proj_kernel(const float* __restrict__ part, int slices, int M, int Sp, const bf16* __restrict__ side, int64_t lds, const int32_t* __restrict__ tok,
+                                                           const bf16* __restrict__ W, int N, bf16* __restrict__ y) {
+    extern __shared__ __attribute__((aligned(16))) bf16 sz[];              // [16][Sp + 8]
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, ld = Sp + 8, n0 = blockIdx.x * 64 + wave * 16;
+    const bf16* w = W + (int64_t)min(n0 + (lane & 15), N - 1) * Sp + (lane >> 4) * 8;
+    bf16x8 wf[8];
+#pragma unroll
+    for (int k = 0; k < 8; k++) wf[k] = *(const bf16x8*)(w + min(k * 32, Sp - 32));      // the first 256 columns travel under z
+    for (int i = tid * 4; i < 16 * Sp; i += 1024) {
+        const int m = i / Sp, n = i - m * Sp;
+        f32x4 z = {0.f, 0.f, 0.f, 0.f};
+        if (m < M) {
+            f32x4 s = {0.f, 0.f, 0.f, 0.f};
+            for (int k = 0; k < slices; k += 8) {
+                f32x4 v[8];
+#pragma unroll
+                for (int q = 0; q < 8; q++) v[q] = k + q < slices ? *(const f32x4*)(part + ((int64_t)(k + q) * M + m) * Sp + n) : f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                for (int q = 0; q < 8; q++) s += v[q];
+            }
+            const f32x4 e = ld4(side + (int64_t)tok[m] * lds + n);
+#pragma unroll
+            for (int q = 0; q < 4; q++) z[q] = gelu_tanh(s[q]) * e[q];
+        }
+        st4(sz + m * ld + n, z);
+    }
+    __syncthreads();
+    const bf16* zr = sz + (lane & 15) * ld + (lane >> 4) * 8;
+    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+    for (int k0 = 0; k0 < Sp; k0 += 256) {
+#pragma unroll
+        for (int k = 0; k < 8; k++)
+            if (k0 + k * 32 < Sp) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[k], *(const bf16x8*)(zr + k0 + k * 32), acc, 0, 0, 0);
+        if (k0 + 256 < Sp) {
+#pragma unroll
+            for (int k = 0; k < 8; k++) wf[k] = *(const bf16x8*)(w + min(k0 + 256 + k * 32, Sp - 32));
+        }
+    }
+    // lane: columns n0 + 4 (lane >> 4) + 0..3 of row lane & 15
+    const int m = lane & 15, n = n0 + 4 * (lane >> 4);
+    if (m < M && n + 4 <= N) *(bf16x4*)(y + (int64_t)m * N + n) = bf16x4{f2bf(acc[0]), f2bf(acc[1]), f2bf(acc[2]), f2bf(acc[3])};
+}
 }  // namespace
 
 int launch_lm_side_act(const Lm& lm, int M, const float* part, int slices, const void* side, int64_t lds, const int32_t* tok, void* z, hipStream_t st) {
     hipLaunchKernelGGL(lm_side_act_kernel, dim3((M * lm.Sp / 4 + 255) / 256), dim3(256), 0, st, part, slices, M, lm.Sp, (const bf16*)side, lds, tok, (bf16*)z);
+    CR_HIP(hipGetLastError());
+    return CR_OK;
+}
+
+bool lm_side_proj_supported(const Lm& lm, int M) { return !lm.f32 && M <= 16 && lm.Sp <= 1024; }
+int launch_lm_side_proj(const Lm& lm, int M, const float* part, int slices, const void* side, int64_t lds, const int32_t* tok, const void* W, void* y, hipStream_t st) {
+    if (!lm_side_proj_supported(lm, M) || M <= 0 || slices <= 0) return cr_fail(CR_ERR_ARG, "token side: %d rows of %d columns", M, lm.Sp);
+    hipLaunchKernelGGL(lm_side_proj_kernel, dim3((lm.Wp + 63) / 64), dim3(256), 16 * (lm.Sp + 8) * 2, st, part, slices, M, lm.Sp, (const bf16*)side, lds, tok, (const bf16*)W, lm.Wp, (bf16*)y);
     CR_HIP(hipGetLastError());
     return CR_OK;
 }

@@ -132,7 +132,7 @@ def test_feed_forward_alone(ff, dtype):
 
 
 @pytest.mark.parametrize('dtype', [F32, BF16])
-@pytest.mark.parametrize('side', [1, 24, 64, 200])
+@pytest.mark.parametrize('side', [1, 24, 64, 200, 300])
 def test_token_side_alone(side, dtype):
     """Three layers, each with its own part of the token's row; prompts and decoding."""
     cfg = LC.config(256, 60, [LC.layer(LC.heads(1, 1, 16, 16, 8), LC.ret(16, 16, (0.9,)), 16 if i else None) for i in range(3)], side=side, loop=(1, 3, 2))
